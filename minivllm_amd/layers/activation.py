@@ -12,6 +12,13 @@ class SiluAndMul(nn.Module):
         return ops.silu_and_mul(x)
 
 
+class GeluTanhAndMul(nn.Module):
+    """``gelu(x[..., :I]) * x[..., I:]`` with the tanh form of gelu, fp32 arithmetic."""
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return ops.gelu_tanh_glu(x, x.dtype)
+
+
 class XIELU(nn.Module):
     """xIELU with two learned numbers p, q: ``softplus(p) z^2 + z/2`` for z > 0 and
     ``(1/2 + softplus(q)) (e^z - 1 - z) + z/2`` otherwise.  The two coefficients are worked out

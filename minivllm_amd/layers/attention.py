@@ -270,44 +270,56 @@ class LatentAttention(nn.Module):
     expansions are never formed: with a_h = W_uk_h^T q_h the score is (a_h . c + q_rot_h . r) *
     scale, and the weighted sum of values is W_uv_h applied to the weighted sum of latents.  So
     this is attention with ONE key/value head whose key row is [c | r] (R + P) and whose value row
-    is c (R), run by ``SinkAttention`` (no sink; its window and kernels), between two batched
-    products per head.  ``up_k`` [H, D, R] and ``up_v`` [H, E, R] are the per-head expansion
-    matrices; ``rotation``: a ``HalfRotation`` over the first entries of the P-part.  Only c and r
+    is c (R), run by ``SinkAttention`` (with its window and sink, when asked for), between two
+    batched products per head.  ``up_k`` [H, D, R] and ``up_v`` [H, R, E] are the per-head
+    expansion matrices, each laid out as the right operand of its product; ``rotation``: a
+    ``HalfRotation`` / ``NeighbourRotation`` over the first entries of the P-part.  Only c and r
     are cached, once: the values are read from the key rows (``value_in_key``)."""
 
     def __init__(self, num_heads: int, head_dim: int, rot_dim: int, v_head_dim: int, kv_rank: int,
-                 scale: float, window: int, rotation, eps: float):
+                 scale: float, window: int, rotation, eps: float, sink: bool = False):
         super().__init__()
         H, D, P, E, R = num_heads, head_dim, rot_dim, v_head_dim, kv_rank
         self.num_heads, self.head_dim, self.rot_dim, self.v_head_dim, self.kv_rank = H, D, P, E, R
         self.eps, self.rotation = eps, rotation
         if rotation.rotary_dim > P:
             raise ValueError("the rotation covers more entries than the rotated part has")
-        self.core = self.make_core(H, P, R, scale, window)
+        self.core = self.make_core(H, P, R, scale, window, sink)
         self.latent_norm = nn.Parameter(torch.ones(R, dtype=torch.float32), requires_grad=False)
         self.up_k = nn.Parameter(torch.zeros(H, D, R), requires_grad=False)
-        self.up_v = nn.Parameter(torch.zeros(H, E, R), requires_grad=False)
+        self.up_v = nn.Parameter(torch.zeros(H, R, E), requires_grad=False)
 
     @staticmethod
-    def make_core(num_heads: int, rot_dim: int, kv_rank: int, scale: float, window: int) -> SinkAttention:
+    def make_core(num_heads: int, rot_dim: int, kv_rank: int, scale: float, window: int,
+                  sink: bool = False) -> SinkAttention:
         """A cache holder of this attention (one per pass of a layer that runs several times):
         one KV head, key rows [c | r], values = the leading R entries of the key rows."""
-        return SinkAttention(num_heads, 1, kv_rank + rot_dim, kv_rank, scale, sink=False,
+        return SinkAttention(num_heads, 1, kv_rank + rot_dim, kv_rank, scale, sink=sink,
                              window=window, value_in_key=True)
+
+    @torch.no_grad()
+    def load_expansions(self, up_k: torch.Tensor, up_v: torch.Tensor, like: torch.Tensor) -> None:
+        """``up_k`` [H*D, R] and ``up_v`` [H*E, R], head by head, as checkpoints hold them."""
+        H, D, E, R = self.num_heads, self.head_dim, self.v_head_dim, self.kv_rank
+        to = dict(device=like.device, dtype=like.dtype)
+        self.up_k = nn.Parameter(up_k.view(H, D, R).to(**to).contiguous(), requires_grad=False)
+        self.up_v = nn.Parameter(up_v.view(H, E, R).transpose(1, 2).to(**to).contiguous(), requires_grad=False)
 
     def forward(self, q: torch.Tensor, dkv: torch.Tensor, core: Optional[SinkAttention] = None
                 ) -> torch.Tensor:
-        """q [T, H, D + P] (the rotated part last), dkv [T, R + P] raw -> [T, H, E] as a
-        transposed view of [H, T, E].  ``core``: the cache holder of this pass (default: the
-        module's own)."""
+        """q [T, H, D + P] (the rotated part last), dkv [T, R + P] raw -> contiguous [T, H, E].
+        ``core``: the cache holder of this pass (default: the module's own)."""
         ctx = get_context()
         core = core or self.core
         T = q.shape[0]
-        H, D, R = self.num_heads, self.head_dim, self.kv_rank
+        H, D, R, E = self.num_heads, self.head_dim, self.kv_rank, self.v_head_dim
         q_abs = torch.bmm(q[:, :, :D].transpose(0, 1), self.up_k)                    # [H, T, R]
         rot = self.rotation
         qf = ops.latent_rope_store(q_abs, q, dkv, self.latent_norm, self.eps, ctx.positions,
                                    rot.inv_freq, rot.rotary_dim, core.k_cache,
-                                   None if core.value_in_key else core.v_cache, ctx.slot_mapping)
+                                   None if core.value_in_key else core.v_cache, ctx.slot_mapping,
+                                   rot.neighbours, rot.mult)
         o = core(qf, None).view(T, H, R)
-        return torch.bmm(o.transpose(0, 1), self.up_v.transpose(1, 2)).transpose(0, 1)   # [T, H, E]
+        out = o.new_empty((T, H, E))
+        torch.bmm(o.transpose(0, 1), self.up_v, out=out.transpose(0, 1))
+        return out

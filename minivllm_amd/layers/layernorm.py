@@ -101,3 +101,20 @@ class ScalarRMSNorm(nn.Module):
 
     def forward(self, x: torch.Tensor, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
         return ops.residual_sum_norm(x, (), (), self.gain, self.eps, out_dtype or x.dtype)
+
+
+class DynamicTanh(nn.Module):
+    """A norm without statistics: ``tanh(alpha x) * weight + bias`` with one number alpha and two
+    vectors, all fp32.  Being element by element it is applied where its input is formed
+    (``ops.hyper_norm``, ``ops.hyper_update_norm``); ``parts`` is what those take."""
+
+    def __init__(self, hidden_size: int):
+        super().__init__()
+        f32 = dict(dtype=torch.float32)
+        self.alpha = nn.Parameter(torch.ones(1, **f32), requires_grad=False)
+        self.weight = nn.Parameter(torch.ones(hidden_size, **f32), requires_grad=False)
+        self.bias = nn.Parameter(torch.zeros(hidden_size, **f32), requires_grad=False)
+
+    @property
+    def parts(self):
+        return self.alpha, self.weight, self.bias

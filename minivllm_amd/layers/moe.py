@@ -122,3 +122,40 @@ class CappedRoutedExperts(nn.Module):
         act = ops.capped_glu_route_scale(F.linear(h, self.gate_up), route, self.ff, self.shared_ff,
                                          self.limit, self.shared_limit, h.dtype, self.slope)
         return F.linear(act, self.down)
+
+
+class CorrectedRoutedExperts(nn.Module):
+    """The capped experts of ``CappedRoutedExperts`` behind another router, with identity experts.
+
+    Router: scores s = softmax(W_r h) in fp32 over the experts and, behind them, ``identity``
+    experts without tensors whose output is the layer's input.  A learned correction is added to
+    the scores for the CHOICE of the ``top`` largest only; the weights are the chosen scores
+    divided by their sum, times ``route_scale``.  A shared expert (own size and limit) runs for
+    every token without a gate.
+
+    Execution as there (stacked projections, zero columns for experts a token did not choose).
+    ``forward`` returns the experts' sum and, when there are identity experts, ``(h, g)`` with
+    g [T] the sum of the identity weights: the caller's stream update adds g h
+    (``ops.hyper_update_norm``), so no separate pass over the row is made for it."""
+
+    def __init__(self, hidden_size: int, ff: int, experts: int, identity: int, top: int, limit: float,
+                 route_scale: float, shared_ff: int = 0, shared_limit: float = 0.0, slope: float = 1.702):
+        super().__init__()
+        if experts < 0 or identity < 0 or not 0 < top <= experts + identity:
+            raise ValueError("router: `top` must lie in 1 .. experts + identity experts")
+        self.slope, self.route_scale = float(slope), float(route_scale)
+        self.ff, self.experts, self.identity, self.top = ff, experts, identity, top
+        self.shared_ff, self.limit, self.shared_limit = shared_ff, float(limit), float(shared_limit)
+        self.columns = experts * ff + shared_ff
+        f32 = dict(dtype=torch.float32)
+        rows = experts + identity
+        self.router = nn.Parameter(torch.zeros(rows, hidden_size, **f32), requires_grad=False)
+        self.correction = nn.Parameter(torch.zeros(rows, **f32), requires_grad=False)
+        self.gate_up = nn.Parameter(torch.zeros(2 * self.columns, hidden_size), requires_grad=False)
+        self.down = nn.Parameter(torch.zeros(hidden_size, self.columns), requires_grad=False)
+
+    def forward(self, h: torch.Tensor):
+        route = ops.corrected_route(h, self.router, self.correction, self.top, self.identity, self.route_scale)
+        act = ops.capped_glu_route_scale(F.linear(h, self.gate_up), route, self.ff, self.shared_ff,
+                                         self.limit, self.shared_limit, h.dtype, self.slope, shared_gate=False)
+        return F.linear(act, self.down), ((h, route[:, self.experts]) if self.identity else None)

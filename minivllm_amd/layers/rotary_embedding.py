@@ -9,6 +9,7 @@ reference's standalone ``(positions, q, k) -> (q, k)`` behaviour.
 """
 from __future__ import annotations
 
+import math
 from functools import lru_cache
 
 import torch
@@ -65,19 +66,48 @@ class PairRotaryEmbedding(nn.Module):
                              persistent=False)
 
 
+def yarn_frequencies(rotary_dim: int, base: float, factor: float, original: float, fast: float,
+                     slow: float):
+    """(frequencies fp64 [rotary_dim/2], factor on cos and sin) of YaRN: a pair that makes more than
+    ``fast`` turns over ``original`` positions keeps its frequency, one that makes fewer than
+    ``slow`` has it divided by ``factor``, a linear ramp over the pair's number in between; cos and
+    sin are multiplied by 0.1 ln(factor) + 1."""
+    i = torch.arange(rotary_dim // 2, dtype=torch.float64)
+    f = base ** (-2.0 * i / rotary_dim)
+
+    def pair_with(turns: float) -> float:
+        return rotary_dim * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+    lo = max(math.floor(pair_with(fast)), 0)
+    hi = min(math.ceil(pair_with(slow)), rotary_dim - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return f / factor * ramp + f * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
+
+
 class HalfRotation(nn.Module):
     """Rotation in the half-split layout on the first ``rotary_dim`` entries of a vector: entry i
     is paired with entry i + rotary_dim/2 and the pair (u, v) at position p becomes
     (u cos a - v sin a, v cos a + u sin a), a = p * base^(-2i / rotary_dim); later entries pass
     unchanged.  Owns only the fp32 frequencies (rounded from float64); the angle is the fp32
     product of position and frequency, formed where the rotation is applied
-    (``ops.latent_rope_store``), so no table and no maximal position."""
+    (``ops.latent_rope_store``), so no table and no maximal position.  ``scaling``: None or YaRN's
+    ``factor / original / fast / slow`` (``mult``: its factor on cos and sin)."""
 
-    def __init__(self, rotary_dim: int, base: float):
+    neighbours = False           # True: entry 2i is paired with entry 2i + 1
+
+    def __init__(self, rotary_dim: int, base: float, scaling=None):
         super().__init__()
         if rotary_dim % 2:
             raise ValueError("rotary_dim must be even")
-        self.rotary_dim, self.base = int(rotary_dim), float(base)
-        i = torch.arange(rotary_dim // 2, dtype=torch.float64)
-        self.register_buffer("inv_freq", (self.base ** (-2.0 * i / max(rotary_dim, 1))).float(),
-                             persistent=False)
+        self.rotary_dim, self.base, self.mult = int(rotary_dim), float(base), 1.0
+        if scaling:
+            f, self.mult = yarn_frequencies(self.rotary_dim, self.base,
+                                            *(float(scaling[k]) for k in ("factor", "original", "fast", "slow")))
+        else:
+            i = torch.arange(rotary_dim // 2, dtype=torch.float64)
+            f = self.base ** (-2.0 * i / max(rotary_dim, 1))
+        self.register_buffer("inv_freq", f.float(), persistent=False)
+
+
+class NeighbourRotation(HalfRotation):
+    """The same in the interleaved layout: entry 2i is paired with entry 2i + 1."""
+    neighbours = True

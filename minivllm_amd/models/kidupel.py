@@ -278,8 +278,7 @@ class KidupelLatentMixer(nn.Module):
         self.q_norm.copy_(_take(w, "dq.norm", (Q,), where))
         self.up_q = _param(_take(w, "uq", (H * (D + P), Q), where), like)
         a.latent_norm.copy_(_take(w, "dkv.norm", (R,), where))
-        a.up_k = _param(_take(w, "uk", (H * D, R), where).view(H, D, R), like)
-        a.up_v = _param(_take(w, "uv", (H * E, R), where).view(H, E, R), like)
+        a.load_expansions(_take(w, "uk", (H * D, R), where), _take(w, "uv", (H * E, R), where), like)
         self.o_proj = _param(_take(w, "o", (W, H * E), where), like)
         return rows, None
 

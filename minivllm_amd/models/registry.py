@@ -114,3 +114,13 @@ def _ensure_builtin() -> None:
         return ZegelixForCausalLM
 
     register(["zegelix"], zegelix_cfg, zegelix_class)
+
+    def danipel_cfg(c, name):
+        from minivllm_amd.models.danipel import DanipelConfig
+        return DanipelConfig.from_dict(c, name)
+
+    def danipel_class():
+        from minivllm_amd.models.danipel import DanipelForCausalLM
+        return DanipelForCausalLM
+
+    register(["danipel"], danipel_cfg, danipel_class)

@@ -395,9 +395,9 @@ def row_norm_store(q, k, v, qw, kw, eps, k_cache, v_cache, slot_mapping):
 
 
 def latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims, k_cache, v_cache,
-                      slot_mapping):
+                      slot_mapping, neighbours=False, mult=1.0):
     return _seqmix(q).latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims,
-                                        k_cache, v_cache, slot_mapping)
+                                        k_cache, v_cache, slot_mapping, neighbours, mult)
 
 
 def xielu(u, ap, aq, out_dtype):
@@ -442,6 +442,24 @@ def rglru_scan(u, gates, gate_bias, lam, y, state, cu_q, positions, slots, sharp
                                  out_dtype)
 
 
-def capped_glu_route_scale(gu, dense, ff, shared_ff, limit, shared_limit, out_dtype, slope=1.702):
+def capped_glu_route_scale(gu, dense, ff, shared_ff, limit, shared_limit, out_dtype, slope=1.702,
+                           shared_gate=True):
     return _seqmix(gu).capped_glu_route_scale(gu, dense, ff, shared_ff, limit, shared_limit, out_dtype,
-                                              slope)
+                                              slope, shared_gate)
+
+
+# ---- several residual streams with a tanh norm, routing with a choice correction, gelu gate
+def hyper_norm(x, read, norm, out_dtype):
+    return _seqmix(x).hyper_norm(x, read, norm, out_dtype)
+
+
+def hyper_update_norm(x, y, skip, write, mix, read, norm, out_dtype):
+    return _seqmix(x).hyper_update_norm(x, y, skip, write, mix, read, norm, out_dtype)
+
+
+def corrected_route(h, router_w, correction, top, identity, scale):
+    return _seqmix(h).corrected_route(h, router_w, correction, top, identity, scale)
+
+
+def gelu_tanh_glu(gu, out_dtype):
+    return _seqmix(gu).gelu_tanh_glu(gu, out_dtype)

@@ -521,21 +521,40 @@ def _rotate_half(x, positions, inv_freq, dims):
     return torch.cat([u * c - v * s, v * c + u * s, x[..., dims:]], -1)
 
 
+def _rotate(x, positions, inv_freq, dims, neighbours=False, mult=1.0):
+    """As ``_rotate_half``; ``neighbours``: entry 2i is paired with entry 2i + 1 instead; cos and sin
+    are multiplied by ``mult``."""
+    if dims == 0:
+        return x
+    half = dims // 2
+    ang = (positions.float()[:, None] * inv_freq.float()[None, :]).double()
+    shape = [x.shape[0]] + [1] * (x.dim() - 2) + [half]
+    c, s = (torch.cos(ang) * mult).float().view(shape), (torch.sin(ang) * mult).float().view(shape)
+    iu = slice(0, dims, 2) if neighbours else slice(0, half)
+    iv = slice(1, dims, 2) if neighbours else slice(half, dims)
+    u, v = x[..., iu], x[..., iv]
+    out = x.clone()
+    out[..., iu] = u * c - v * s
+    out[..., iv] = v * c + u * s
+    return out
+
+
 def latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims, k_cache, v_cache,
-                      slot_mapping):
+                      slot_mapping, neighbours=False, mult=1.0):
     """Assembles the queries and cache rows of attention over a shared latent.  ``q_abs`` [H,T,R]:
     the heads' unrotated query parts carried into the latent's coordinates; ``q`` [T,H,D+P] whose
     last P entries per head are the part to rotate; ``dkv`` [T,R+P]: the raw latent and one key
     part shared by all heads.  K cache row = [rmsnorm(latent) * w | rotated key part] (one KV
     head of R + P), V cache row = the normed latent (R; ``v_cache`` None: not written, the reader
     takes the leading R entries of the key rows).  Returns the queries [T,H,R+P] =
-    [q_abs | rotated part].  The rotation turns the first ``rot_dims`` of the P entries."""
+    [q_abs | rotated part].  The rotation turns the first ``rot_dims`` of the P entries in
+    half-split pairs, or in pairs of ``neighbours``, cos and sin both times ``mult``."""
     H, T, R = q_abs.shape
     P = dkv.shape[1] - R
     D = q.shape[2] - P
     c = rms_norm_rows(dkv[:, :R], w, eps, torch.float32)
-    kr = _rotate_half(dkv[:, R:].float(), positions, inv_freq, rot_dims)
-    qr = _rotate_half(q[:, :, D:].float(), positions, inv_freq, rot_dims)
+    kr = _rotate(dkv[:, R:].float(), positions, inv_freq, rot_dims, neighbours, mult)
+    qr = _rotate(q[:, :, D:].float(), positions, inv_freq, rot_dims, neighbours, mult)
     out = torch.cat([q_abs.transpose(0, 1).float(), qr], -1).to(q.dtype)
     if k_cache is not None and slot_mapping is not None:
         _scatter_rows(k_cache, torch.cat([c, kr], -1)[:, None, :], slot_mapping)
@@ -682,13 +701,14 @@ def rglru_scan(u, gates, gate_bias, lam, y, state, cu_q, positions, slots, sharp
     return (out * gelu_tanh(y.float())).to(out_dtype)
 
 
-def capped_glu_route_scale(gu, dense, ff, shared_ff, limit, shared_limit, out_dtype, slope=1.702):
+def capped_glu_route_scale(gu, dense, ff, shared_ff, limit, shared_limit, out_dtype, slope=1.702,
+                           shared_gate=True):
     """gu [T, 2 C], C = experts * ff + shared_ff: the gate projections of all experts (and of a
     shared one behind them), then their up projections.  Column c: g = min(gate, L), u =
     clamp(up, -L, L), act = w g sigmoid(slope g) (u + 1) with L = ``limit`` for routed columns and
     ``shared_limit`` for shared ones, w = dense[t, expert] for routed columns (exactly zero where w
-    is) and, for shared columns, dense[t, experts] when ``dense`` has that extra column (a
-    per-token gate of the shared expert), else 1.  Returns [T, C]."""
+    is) and, for shared columns, dense[t, experts] when ``dense`` has that extra column and
+    ``shared_gate`` says it is a per-token gate of the shared expert, else 1.  Returns [T, C]."""
     T, C = gu.shape[0], gu.shape[1] // 2
     ne = (C - shared_ff) // ff if ff else 0
     g, u = gu[:, :C].float(), gu[:, C:2 * C].float()
@@ -696,6 +716,57 @@ def capped_glu_route_scale(gu, dense, ff, shared_ff, limit, shared_limit, out_dt
     g = torch.minimum(g, lim)
     u = torch.maximum(torch.minimum(u, lim), -lim)
     act = g * torch.sigmoid(slope * g) * (u + 1.0)
-    sg = dense[:, ne:ne + 1].float() if dense.shape[1] > ne else torch.ones(T, 1)
+    sg = dense[:, ne:ne + 1].float() if shared_gate and dense.shape[1] > ne else torch.ones(T, 1)
     w = torch.cat([dense[:, :ne].float().repeat_interleave(ff, 1), sg.expand(T, shared_ff)], 1)
     return torch.where(w != 0, act * w, torch.zeros_like(act)).to(out_dtype)
+
+
+# ------------------------------------------------------------------ several residual streams
+def _tanh_norm(u, norm, out_dtype):
+    alpha, w, b = norm
+    return (torch.tanh(alpha.float() * u) * w.float() + b.float()).to(out_dtype)
+
+
+def hyper_norm(x, read, norm, out_dtype):
+    """x [T, S, W] fp32 residual streams (the S rows of a token may be one row seen S times: a
+    zero stride) -> tanh(alpha u) * w + b of u = sum_s read[s] x_s.  ``norm`` = (alpha [1], w [W],
+    b [W]), all fp32."""
+    return _tanh_norm((x * read.float()[None, :, None]).sum(1), norm, out_dtype)
+
+
+def hyper_update_norm(x, y, skip, write, mix, read, norm, out_dtype):
+    """Every stream from the old ones: x_b <- sum_a mix[a, b] x_a + write[b] (y + g h), in place
+    (or into a new tensor when the streams of x are one row seen S times).  ``skip``: None or
+    (h [T, W], g [T]) - a multiple per token of the sublayer's input that joins its output.
+    Returns (streams, next input): with ``read`` / ``norm`` given the next sublayer's
+    input is ``hyper_norm`` of the new streams, else None."""
+    t = y.float()
+    if skip is not None:
+        t = t + skip[1].float()[:, None] * skip[0].float()
+    new = torch.einsum("ab,taw->tbw", mix.float(), x) + write.float()[None, :, None] * t[:, None, :]
+    if x.stride(1) == 0 and x.shape[1] > 1:
+        x = new
+    else:
+        x.copy_(new)
+    return x, (hyper_norm(x, read, norm, out_dtype) if read is not None else None)
+
+
+# ------------------------------------------------------------------ corrected routing, gelu gate
+def corrected_route(h, router_w, correction, top, identity, scale):
+    """Scores = softmax over all rows of ``router_w`` (fp32), the last ``identity`` of which are
+    identity experts.  The ``top`` largest score + correction are chosen (ties to the lower
+    index); their weights are their scores without the correction, divided by their sum (+ 1e-20),
+    times ``scale``.  Returns [T, experts + 1] fp32: the experts' weights (zero where not
+    chosen), then the sum of the chosen identity experts' weights."""
+    s = torch.softmax(h.float() @ router_w.float().t(), -1)
+    ids = torch.sort(s + correction.float(), dim=-1, descending=True, stable=True).indices[:, :top]
+    p = s.gather(1, ids)
+    full = torch.zeros_like(s).scatter_(1, ids, p / (p.sum(-1, keepdim=True) + 1e-20) * scale)
+    n = s.shape[1] - identity
+    return torch.cat([full[:, :n], full[:, n:].sum(-1, keepdim=True)], 1)
+
+
+def gelu_tanh_glu(gu, out_dtype):
+    """gu [T, 2 C] (gate columns, then up columns; rows may be strided) -> gelu_tanh(gate) * up."""
+    C = gu.shape[1] // 2
+    return (gelu_tanh(gu[:, :C].float()) * gu[:, C:].float()).to(out_dtype)
