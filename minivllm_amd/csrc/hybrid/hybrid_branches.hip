@@ -93,8 +93,22 @@ __global__ void row_norm_store_kernel(T* __restrict__ q, const T* __restrict__ k
 // Per token: c = rmsnorm(dkv[0:R]) * w;  K cache row = [c | rot(dkv[R:R+P])], V cache row = c
 // (when a separate V cache is given);
 // out[t, h] = [q_abs[h, t, 0:R] | rot(q[t, h, D:D+P])].  rot: entry i < dims/2 pairs with entry
-// i + dims/2, angle = position * inv_freq[i] (fp32 product), entries from dims on unchanged.
+// i + dims/2 (neighbours: entry 2i with entry 2i + 1), angle = position * inv_freq[i] (fp32
+// product), cos and sin times mult, entries from dims on unchanged.
 template <typename T>
+__device__ __forceinline__ float turned(const T* r, int i, int dims, int neighbours, const float* cs,
+                                        const float* sn) {
+    const int half = dims >> 1;
+    if (i >= dims) return ld(r + i);
+    if (neighbours) {
+        const float c = cs[i >> 1], s = sn[i >> 1];
+        return (i & 1) ? ld(r + i) * c + ld(r + i - 1) * s : ld(r + i) * c - ld(r + i + 1) * s;
+    }
+    return i < half ? ld(r + i) * cs[i] - ld(r + i + half) * sn[i]
+                    : ld(r + i) * cs[i - half] + ld(r + i - half) * sn[i - half];
+}
+
+template <typename T, int VEC>
 __global__ void latent_rope_store_kernel(const T* __restrict__ q_abs, const T* __restrict__ q,
                                          long q_row, const T* __restrict__ dkv, long dkv_row,
                                          const float* __restrict__ w, float eps,
@@ -102,7 +116,8 @@ __global__ void latent_rope_store_kernel(const T* __restrict__ q_abs, const T* _
                                          const float* __restrict__ inv_freq, int dims,
                                          T* __restrict__ k_cache, T* __restrict__ v_cache,
                                          const int* __restrict__ slot_mapping, T* __restrict__ out,
-                                         long T_, int H, int D, int P, int R) {
+                                         long T_, int H, int D, int P, int R, int neighbours,
+                                         float mult) {
     extern __shared__ float sm[];            // [dims/2] cos, [dims/2] sin, then 16 for sums
     const int half = dims / 2;
     float* cs = sm;
@@ -115,7 +130,7 @@ __global__ void latent_rope_store_kernel(const T* __restrict__ q_abs, const T* _
     for (int i = threadIdx.x; i < half; i += blockDim.x) {
         float s_, c_;
         sincosf(p * inv_freq[i], &s_, &c_);
-        cs[i] = c_; sn[i] = s_;
+        cs[i] = c_ * mult; sn[i] = s_ * mult;
     }
     const T* lr = dkv + t * dkv_row;
     float ss = 0.f;
@@ -128,26 +143,33 @@ __global__ void latent_rope_store_kernel(const T* __restrict__ q_abs, const T* _
             st(k_cache + slot * DK + c, a);
             if (v_cache) st(v_cache + slot * R + c, a);   // null: values are read from the key rows
         }
-        for (int i = threadIdx.x; i < P; i += blockDim.x) {
-            float a;
-            if (i < half) a = ld(lr + R + i) * cs[i] - ld(lr + R + i + half) * sn[i];
-            else if (i < dims) a = ld(lr + R + i) * cs[i - half] + ld(lr + R + i - half) * sn[i - half];
-            else a = ld(lr + R + i);
-            st(k_cache + slot * DK + R + i, a);
-        }
+        for (int i = threadIdx.x; i < P; i += blockDim.x)
+            st(k_cache + slot * DK + R + i, turned(lr + R, i, dims, neighbours, cs, sn));
     }
-    for (int j = threadIdx.x; j < H * DK; j += blockDim.x) {
+    // the queries: VEC entries per thread and step (VEC = 8: R, P and the rows are whole runs)
+    for (int j = threadIdx.x * VEC; j < H * DK; j += blockDim.x * VEC) {
         const int hh = j / DK, c = j - hh * DK;
-        float a;
-        if (c < R) a = ld(q_abs + ((long)hh * T_ + t) * R + c);
-        else {
-            const T* qr = q + t * q_row + (long)hh * (D + P) + D;
-            const int i = c - R;
-            if (i < half) a = ld(qr + i) * cs[i] - ld(qr + i + half) * sn[i];
-            else if (i < dims) a = ld(qr + i) * cs[i - half] + ld(qr + i - half) * sn[i - half];
-            else a = ld(qr + i);
+        T* dst = out + t * (long)(H * DK) + j;
+        if constexpr (VEC == 8) {
+            if (c < R) {
+                const T* src = q_abs + ((long)hh * T_ + t) * R + c;
+                if constexpr (sizeof(T) == 2) {
+                    *reinterpret_cast<uint4*>(dst) = *reinterpret_cast<const uint4*>(src);
+                } else {
+                    *reinterpret_cast<float4*>(dst) = *reinterpret_cast<const float4*>(src);
+                    *reinterpret_cast<float4*>(dst + 4) = *reinterpret_cast<const float4*>(src + 4);
+                }
+            } else {
+                const T* qr = q + t * q_row + (long)hh * (D + P) + D;
+                float a[8];
+#pragma unroll
+                for (int e = 0; e < 8; ++e) a[e] = turned(qr, c - R + e, dims, neighbours, cs, sn);
+                store_run8<T>(dst, a);
+            }
+        } else {
+            st(dst, c < R ? ld(q_abs + ((long)hh * T_ + t) * R + c)
+                          : turned(q + t * q_row + (long)hh * (D + P) + D, c - R, dims, neighbours, cs, sn));
         }
-        st(out + t * (long)(H * DK) + j, a);
     }
 }
 
@@ -272,17 +294,22 @@ int hyb_latent_rope_store(const void* q_abs, const void* q, long q_row, const vo
                           long dkv_row, const void* w, float eps, const void* positions,
                           const void* inv_freq, int dims, void* k_cache, void* v_cache,
                           const void* slot_mapping, void* out, long T_, int H, int D, int P, int R,
-                          int dt, hipStream_t s) {
+                          int neighbours, float mult, int dt, hipStream_t s) {
     if (T_ <= 0) return 0;
     if (dims < 0 || (dims & 1) || dims > P || H <= 0 || R <= 0) return 1;
     const size_t lds = (dims + 16) * sizeof(float);
     if (lds > 64 * 1024) return 1;
-    HYB_DISPATCH(dt, hipLaunchKernelGGL(latent_rope_store_kernel<T>, dim3(T_),
-                                        dim3(threads_for(H * (R + P))), lds, s, (const T*)q_abs,
-                                        (const T*)q, q_row, (const T*)dkv, dkv_row, (const float*)w,
-                                        eps, (const int*)positions, (const float*)inv_freq, dims,
-                                        (T*)k_cache, (T*)v_cache, (const int*)slot_mapping, (T*)out,
-                                        T_, H, D, P, R));
+    const bool vec = R % 8 == 0 && P % 8 == 0 && (size_t)q_abs % 16 == 0 && (size_t)out % 16 == 0;
+#define LRS(VEC)                                                                                   \
+    HYB_DISPATCH(dt, hipLaunchKernelGGL((latent_rope_store_kernel<T, VEC>), dim3(T_),              \
+                                        dim3(threads_for(H * (R + P) / VEC)), lds, s,              \
+                                        (const T*)q_abs, (const T*)q, q_row, (const T*)dkv, dkv_row, \
+                                        (const float*)w, eps, (const int*)positions,               \
+                                        (const float*)inv_freq, dims, (T*)k_cache, (T*)v_cache,    \
+                                        (const int*)slot_mapping, (T*)out, T_, H, D, P, R,         \
+                                        neighbours, mult))
+    if (vec) LRS(8); else LRS(1);
+#undef LRS
     return HYB_LAUNCH_OK();
 }
 

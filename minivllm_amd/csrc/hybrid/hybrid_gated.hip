@@ -431,20 +431,20 @@ __global__ void chosen_route_kernel(const T* __restrict__ h, const float* __rest
     }
 }
 
-// gu row = [gate columns C | up columns C], C = NE * ff + sff; dense [T, NR], NR = NE (+ 1: the
-// shared columns' gate).  VEC consecutive columns per thread (VEC divides ff, sff, the strides).
+// gu row = [gate columns C | up columns C], C = NE * ff + sff; dense [T, NR]; sgate: column NE of
+// it gates the shared columns (else they are taken as they are).  VEC consecutive columns per thread (VEC divides ff, sff, the strides).
 template <typename T, int VEC>
 __global__ void capped_glu_route_scale_kernel(const T* __restrict__ gu, long gu_stride,
                                               const float* __restrict__ dense, T* __restrict__ act,
                                               int NE, int NR, int ff, int C, float limit,
-                                              float shared_limit, float slope) {
+                                              float shared_limit, float slope, int sgate) {
     const long t = blockIdx.y;
     const T* g = gu + t * gu_stride;
     const T* u = g + C;
     const int routed = NE * ff;
     for (int c = (blockIdx.x * blockDim.x + threadIdx.x) * VEC; c < C; c += gridDim.x * blockDim.x * VEC) {
         const bool sh = c >= routed;
-        const float w = sh ? (NR > NE ? dense[t * NR + NE] : 1.f) : dense[t * NR + c / ff];
+        const float w = sh ? (sgate ? dense[t * NR + NE] : 1.f) : dense[t * NR + c / ff];
         const float L = sh ? shared_limit : limit;
         float gv[VEC], uv[VEC];
         if (w != 0.f) {
@@ -579,10 +579,10 @@ int hyb_chosen_route(const void* h, const void* wr, const void* bias, void* dens
 
 int hyb_capped_glu_route_scale(const void* gu, long gu_stride, const void* dense, void* act, long T_,
                                int NE, int NR, int ff, int sff, float limit, float shared_limit,
-                               float slope, int dt, hipStream_t s) {
+                               float slope, int sgate, int dt, hipStream_t s) {
     const int C = NE * ff + sff;
     if (T_ <= 0 || C <= 0) return 0;
-    if (!dense || NR < NE) return 1;
+    if (!dense || NR < NE || (sgate && NR == NE)) return 1;
     const int esize = dt == 0 ? 2 : 4;
     const bool vec = (NE == 0 || ff % 8 == 0) && sff % 8 == 0 && gu_stride % 8 == 0 &&
                      (size_t)gu % (4 * esize) == 0 && (C * (size_t)esize) % (4 * esize) == 0;
@@ -596,7 +596,7 @@ int hyb_capped_glu_route_scale(const void* gu, long gu_stride, const void* dense
                                             dim3(256), 0, s, (const T*)gu + t0 * gu_stride,       \
                                             gu_stride, (const float*)dense + t0 * NR,             \
                                             (T*)act + t0 * (long)C, NE, NR, ff, C, limit,         \
-                                            shared_limit, slope))
+                                            shared_limit, slope, sgate))
         if (vec) CGLU(8); else CGLU(1);
 #undef CGLU
     }

@@ -69,7 +69,7 @@ _rsn = _sig("hyb_residual_sum_norm", _P, _P, _P, _P, _I, _F, _P, _L, _I, _F, _I,
 _rnr = _sig("hyb_rms_norm_rows", _P, _L, _P, _P, _L, _I, _F, _I, _P)
 _rns = _sig("hyb_row_norm_store", _P, _P, _P, _L, _P, _P, _F, _P, _P, _P, _L, _I, _I, _I, _I, _P)
 _lrs = _sig("hyb_latent_rope_store", _P, _P, _L, _P, _L, _P, _F, _P, _P, _I, _P, _P, _P, _P, _L, _I,
-            _I, _I, _I, _I, _P)
+            _I, _I, _I, _I, _F, _I, _P)
 _xie = _sig("hyb_xielu", _P, _L, _P, _L, _I, _F, _F, _I, _P)
 _ggn = _sig("hyb_gated_group_norm", _P, _P, _P, _P, _L, _P, _P, _L, _I, _I, _I, _F, _I, _P)
 _sgt = _sig("hyb_sigmoid_gate", _P, _L, _L, _P, _L, _P, _L, _I, _I, _I, _P)
@@ -79,7 +79,11 @@ _utg = _sig("hyb_unturn_gate", _P, _L, _L, _P, _P, _P, _L, _P, _L, _I, _I, _I, _
 _scv = _sig("hyb_short_conv", _P, _L, _P, _P, _P, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _P)
 _lru = _sig("hyb_rglru_scan", _P, _P, _P, _P, _P, _L, _P, _P, _P, _P, _P, _L, _I, _I, _I, _F, _I, _I, _P)
 _crt = _sig("hyb_chosen_route", _P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _P)
-_cgl = _sig("hyb_capped_glu_route_scale", _P, _L, _P, _P, _L, _I, _I, _I, _I, _F, _F, _F, _I, _P)
+_cgl = _sig("hyb_capped_glu_route_scale", _P, _L, _P, _P, _L, _I, _I, _I, _I, _F, _F, _F, _I, _I, _P)
+_hyp = _sig("hyb_hyper_update_norm", _P, _L, _L, _P, _P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _P, _P, _P, _L, _I,
+            _I, _I, _P)
+_cor = _sig("hyb_corrected_route", _P, _P, _P, _P, _L, _I, _I, _I, _I, _F, _I, _P)
+_gtg = _sig("hyb_gelu_tanh_glu", _P, _L, _P, _L, _I, _I, _P)
 
 _DT = {torch.bfloat16: 0, torch.float32: 2}
 
@@ -597,7 +601,7 @@ def row_norm_store(q, k, v, qw, kw, eps, k_cache, v_cache, slot_mapping):
 
 
 def latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims, k_cache, v_cache,
-                      slot_mapping):
+                      slot_mapping, neighbours=False, mult=1.0):
     H, T, R = q_abs.shape
     P = dkv.shape[1] - R
     D = q.shape[2] - P
@@ -612,7 +616,7 @@ def latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims, k_ca
     _check(_lrs(q_abs.data_ptr(), q.data_ptr(), _rows(q), dkv.data_ptr(), _rows(dkv),
                 _f32(w).data_ptr(), eps, _i32(positions).data_ptr(), _f32(inv_freq).data_ptr(),
                 int(rot_dims), _ptr(k_cache), _ptr(v_cache), _ptr(_i32(slot_mapping)), out.data_ptr(),
-                T, H, D, P, R, _dt(q), _stream()), "latent_rope_store")
+                T, H, D, P, R, int(neighbours), float(mult), _dt(q), _stream()), "latent_rope_store")
     return out
 
 
@@ -739,14 +743,80 @@ def rglru_scan(u, gates, gate_bias, lam, y, state, cu_q, positions, slots, sharp
     return out
 
 
-def capped_glu_route_scale(gu, dense, ff, shared_ff, limit, shared_limit, out_dtype, slope=1.702):
+def capped_glu_route_scale(gu, dense, ff, shared_ff, limit, shared_limit, out_dtype, slope=1.702,
+                           shared_gate=True):
     T = gu.shape[0]
     C = gu.shape[1] // 2
     NR = dense.shape[1]
-    NE = (C - shared_ff) // ff
+    NE = (C - shared_ff) // ff if ff else 0
     assert gu.stride(1) == 1 and gu.dtype == out_dtype and C == NE * ff + shared_ff and NR in (NE, NE + 1)
     act = torch.empty((T, C), dtype=out_dtype, device=gu.device)
     _check(_cgl(gu.data_ptr(), _rows(gu), _f32(dense).data_ptr(), act.data_ptr(), T, NE, NR, ff,
-                shared_ff, float(limit), float(shared_limit), float(slope), _dt(gu), _stream()),
+                shared_ff, float(limit), float(shared_limit), float(slope),
+                int(bool(shared_gate) and NR > NE), _dt(gu), _stream()),
            "capped_glu_route_scale")
+    return act
+
+
+# ------------------------------------------------------------------ several residual streams
+def _streams_of(x):
+    """(streams, elements from one stream of a token to the next); rows dense."""
+    assert x.dtype == torch.float32 and x.dim() == 3 and x.stride(2) == 1
+    return x.shape[1], (x.stride(1) if x.shape[1] > 1 else x.shape[2])
+
+
+def _norm_ptrs(read, norm, S, W):
+    if read is None:
+        return (None,) * 4
+    alpha, w, b = norm
+    assert read.numel() == S and w.numel() == W and b.numel() == W and alpha.numel() == 1
+    return tuple(_f32(t).data_ptr() for t in (read, alpha, w, b))
+
+
+def hyper_norm(x, read, norm, out_dtype):
+    T, S, W = x.shape
+    _, xs = _streams_of(x)
+    h = torch.empty((T, W), dtype=out_dtype, device=x.device)
+    _check(_hyp(x.data_ptr(), x.stride(0), xs, None, None, 0, None, 0, None, 0, None, None,
+                *_norm_ptrs(read, norm, S, W), h.data_ptr(), T, S, W, _DT[out_dtype], _stream()),
+           "hyper_norm")
+    return h
+
+
+def hyper_update_norm(x, y, skip, write, mix, read, norm, out_dtype):
+    T, S, W = x.shape
+    _, xs = _streams_of(x)
+    assert y.shape == (T, W) and y.stride(1) == 1 and y.dtype == out_dtype
+    assert write.numel() == S and mix.shape == (S, S)
+    hs = gs = None
+    if skip is not None:
+        hs, gs = skip
+        assert hs.shape == (T, W) and hs.stride(1) == 1 and hs.dtype == out_dtype
+        assert gs.shape == (T,) and gs.dtype == torch.float32
+    in_place = x.is_contiguous()
+    new = x if in_place else torch.empty((T, S, W), dtype=torch.float32, device=x.device)
+    h = torch.empty((T, W), dtype=out_dtype, device=x.device) if read is not None else None
+    _check(_hyp(x.data_ptr(), x.stride(0) if not in_place else S * W, xs, new.data_ptr(), y.data_ptr(),
+                _rows(y), _ptr(hs), _rows(hs) if hs is not None else 0, _ptr(gs),
+                gs.stride(0) if gs is not None else 0, _f32(write).data_ptr(), _f32(mix).data_ptr(),
+                *_norm_ptrs(read, norm, S, W), _ptr(h), T, S, W, _DT[out_dtype], _stream()),
+           "hyper_update_norm")
+    return new, h
+
+
+def corrected_route(h, router_w, correction, top, identity, scale):
+    T, W = h.shape
+    NR = router_w.shape[0]
+    assert h.is_contiguous() and router_w.shape[1] == W and correction.numel() == NR and 0 <= identity <= NR
+    dense = torch.empty((T, NR - identity + 1), dtype=torch.float32, device=h.device)
+    _check(_cor(h.data_ptr(), _f32(router_w).data_ptr(), _f32(correction).data_ptr(), dense.data_ptr(),
+                T, W, NR - identity, NR, int(top), float(scale), _dt(h), _stream()), "corrected_route")
+    return dense
+
+
+def gelu_tanh_glu(gu, out_dtype):
+    T, C = gu.shape[0], gu.shape[1] // 2
+    assert gu.stride(1) == 1 and gu.dtype == out_dtype and gu.shape[1] == 2 * C
+    act = torch.empty((T, C), dtype=out_dtype, device=gu.device)
+    _check(_gtg(gu.data_ptr(), _rows(gu), act.data_ptr(), T, C, _dt(gu), _stream()), "gelu_tanh_glu")
     return act
