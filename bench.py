@@ -386,6 +386,32 @@ def zegelix_model(size: str, vocab: int = 32768, experts: int = 4, top: int = 2,
                                     "loop": {"start": 1, "stop": 3, "times": 2}}, name=f"zegelix-{size}")
 
 
+def danipel_model(size: str, vocab: int = 32768, experts: int = 4, identity: int = 2, top: int = 2):
+    """Danipel configuration of the same width, number of layer runs, heads and active feed-forward
+    parameters per token as ``hybrid_models(size)``: eight layers, the two kinds of latent
+    attention in turn with DeepSeek's proportions (latent of 512 + a rotated part of 64, heads of
+    128 + 64 on the query side and 128 values, queries of the second kind through a latent of
+    3 W / 8), full causal attention, two residual streams; a dense layer first, then routed
+    clamped experts plus a shared one ((top + 1) * 3 * ff = 3 * intermediate) with identity
+    experts behind them."""
+    from minivllm_amd.models.danipel import DanipelConfig
+    W, L, H, G, D, inter = HYBRID_SIZES[size]
+    ff = inter // (top + 1) // 64 * 64
+    moe = {"kind": "moe", "expert": {"ff": ff, "limit": 7.0},
+           "router": {"experts": experts, "identity": identity, "top": top, "scale": 2.5},
+           "shared": {"ff": ff, "limit": 7.0}}
+    m = {"heads": H, "dim": D, "rot_dim": 64, "vdim": D, "kv_rank": 512, "scale": (D + 64) ** -0.5}
+    yarn = {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}
+    kinds = [("latent_attention_2", dict(m, q_rank=3 * W // 8, rot={"base": 10000.0, "dims": 64})),
+             ("latent_attention", dict(m, rot={"base": 10000.0, "dims": 64, "scaling": yarn}))]
+    layers = [{"type": kinds[i % 2][0], "mixer": kinds[i % 2][1],
+               "mlp": moe if i else {"kind": "dense", "ff": inter}} for i in range(L)]
+    return DanipelConfig.from_dict({"architecture": "Danipel", "vocab": vocab, "width": W,
+                                    "norm": {"eps": 1e-6}, "embedding": {"scale": float(W) ** 0.5},
+                                    "residual_mult": 1.0, "streams": 2, "layers": layers},
+                                   name=f"danipel-{size}")
+
+
 def hybrid_comparison(args) -> dict:
     """Prefill and decode throughput of the hybrid families next to the dense decoder of the same
     size, one GPU, same engine path as the headline measurement (``bench_model``).
@@ -397,6 +423,8 @@ def hybrid_comparison(args) -> dict:
         return kidupel_comparison(args)
     if args.family == "zegelix":
         return zegelix_comparison(args)
+    if args.family == "danipel":
+        return danipel_comparison(args)
     out = {"metric": "prefill / decode tok/s, hybrid (attention + delta rule + routed experts) "
                      "next to the dense decoder of equal size",
            "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
@@ -499,6 +527,34 @@ def zegelix_comparison(args) -> dict:
             if all(n in row and k in row[n] for n in ("zegelix", "kidupel", "dense")):
                 row[f"zegelix_over_kidupel_{k}"] = round(row["zegelix"][k] / row["kidupel"][k], 3)
                 row[f"zegelix_over_dense_{k}"] = round(row["zegelix"][k] / row["dense"][k], 3)
+        out["sizes"][size] = row
+    return out
+
+
+def danipel_comparison(args) -> dict:
+    out = {"metric": "prefill / decode tok/s, Danipel (two kinds of latent attention, hyper-connected "
+                     "residual streams, tanh norms, corrected routing with identity experts) next "
+                     "to Kidupel and the dense decoder of equal size",
+           "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+           "dtype": "bf16", "data": "synthetic random token prompts, random-init weights",
+           "config": {"seq_len": args.seq_len, "decode_batch": args.batch,
+                      "prefill_tokens_per_step": args.prefill_tokens, "kv_block_size": args.block_size},
+           "sizes": {}}
+    keep = ("prefill_tok_s", "prefill_ms_per_step", "decode_tok_s", "decode_ms_per_step",
+            "hipgraph_captured", "init_s")
+    for size in args.hybrid.split(","):
+        _, dense = hybrid_models(size)
+        row = {}
+        for name, make in (("danipel", lambda: danipel_model(size)), ("kidupel", lambda: kidupel_model(size)),
+                           ("dense", lambda: dense)):
+            if args.only and name != args.only:
+                continue                         # (a kernel trace of one model)
+            r = bench_model(args, make(), 0, 1)
+            row[name] = {k: (round(v, 3) if isinstance(v, float) else v) for k, v in r.items() if k in keep}
+        for k in ("prefill_tok_s", "decode_tok_s"):
+            if all(n in row and k in row[n] for n in ("danipel", "kidupel", "dense")):
+                row[f"danipel_over_kidupel_{k}"] = round(row["danipel"][k] / row["kidupel"][k], 3)
+                row[f"danipel_over_dense_{k}"] = round(row["danipel"][k] / row["dense"][k], 3)
         out["sizes"][size] = row
     return out
 
@@ -802,12 +858,12 @@ def main():
                          "launch floor of a real N-GPU run; NOT a scaling number)")
     ap.add_argument("--p2p", action="store_true",
                     help="with --tp-shard: all-reduces by the peer-to-peer kernels in loop-back form")
-    ap.add_argument("--family", default="natilix", choices=["natilix", "pelenex", "kidupel", "zegelix"],
+    ap.add_argument("--family", default="natilix", choices=["natilix", "pelenex", "kidupel", "zegelix", "danipel"],
                     help="with --hybrid: which hybrid family is measured (pelenex: next to natilix "
-                         "and dense; kidupel: next to pelenex and dense; zegelix: next to kidupel "
-                         "and dense)")
-    ap.add_argument("--only", default="", choices=["", "zegelix", "kidupel", "pelenex", "natilix", "dense"],
-                    help="with --hybrid --family pelenex / kidupel: measure this one model only")
+                         "and dense; kidupel: next to pelenex and dense; zegelix, danipel: next to "
+                         "kidupel and dense)")
+    ap.add_argument("--only", default="", choices=["", "danipel", "zegelix", "kidupel", "pelenex", "natilix", "dense"],
+                    help="with --hybrid --family pelenex / kidupel / zegelix / danipel: measure this one model only")
     ap.add_argument("--hybrid", default="",
                     help="instead of the headline workload: the hybrid family (Natilix) next to "
                          "the dense decoder of equal size; comma-separated sizes of "

@@ -25,11 +25,9 @@
 // allocations as the token rows, pool_base rows behind their start: pooled row b of a sequence is
 // row pool_base + table[b / pool_rows] * pool_rows + b % pool_rows.  In the order the kernels walk
 // a query's keys the pooled rows come first, then the window's tokens.
-#include "hybrid_common.h"
+#include "hybrid_merge.h"
 
 using namespace hyb;
-
-constexpr float NO_SINK_MAX = -1e30f;
 
 struct KeyRule {
     int window;             // 0: every earlier key is visible
@@ -606,29 +604,6 @@ sink_attention_split_kernel(const T* __restrict__ q, long q_row, long q_head,
             }
         }
         ws[(((long)b * H + h0 + r) * splits + split) * PS + x] = v;
-    }
-}
-
-template <typename T>
-__global__ void sink_attention_merge_kernel(const float* __restrict__ ws,
-                                            const float* __restrict__ sink,
-                                            const T* __restrict__ gate, long gate_row,
-                                            const int* __restrict__ context_lens,
-                                            T* __restrict__ out, int H, int E, int splits) {
-    const int b = blockIdx.x / H, h = blockIdx.x % H;
-    if (context_lens[b] <= 0) return;
-    const int PS = E + 2;
-    const float* p = ws + ((long)b * H + h) * splits * PS;
-    float M = sink ? sink[h] : NO_SINK_MAX;
-    for (int s = 0; s < splits; ++s) M = fmaxf(M, p[s * PS]);
-    float L = sink ? expf(sink[h] - M) : 0.f;
-    for (int s = 0; s < splits; ++s) L += p[s * PS + 1] * expf(p[s * PS] - M);
-    float f = 1.f / L;
-    if (gate) f *= sigmoidf_(ld(gate + b * gate_row + h));
-    for (int e = threadIdx.x; e < E; e += blockDim.x) {
-        float v = 0.f;
-        for (int s = 0; s < splits; ++s) v += p[s * PS + 2 + e] * expf(p[s * PS] - M);
-        st(out + ((long)b * H + h) * E + e, v * f);
     }
 }
 

@@ -92,7 +92,7 @@ __global__ void row_norm_store_kernel(T* __restrict__ q, const T* __restrict__ k
 
 // Per token: c = rmsnorm(dkv[0:R]) * w;  K cache row = [c | rot(dkv[R:R+P])], V cache row = c
 // (when a separate V cache is given);
-// out[t, h] = [q_abs[h, t, 0:R] | rot(q[t, h, D:D+P])].  rot: entry i < dims/2 pairs with entry
+// out[t, h] = [q_abs[h, t, 0:R] | rot(q[t, h, D:D+P])] (q_abs null: the rotated part alone).  rot: entry i < dims/2 pairs with entry
 // i + dims/2 (neighbours: entry 2i with entry 2i + 1), angle = position * inv_freq[i] (fp32
 // product), cos and sin times mult, entries from dims on unchanged.
 template <typename T>
@@ -147,9 +147,10 @@ __global__ void latent_rope_store_kernel(const T* __restrict__ q_abs, const T* _
             st(k_cache + slot * DK + R + i, turned(lr + R, i, dims, neighbours, cs, sn));
     }
     // the queries: VEC entries per thread and step (VEC = 8: R, P and the rows are whole runs)
-    for (int j = threadIdx.x * VEC; j < H * DK; j += blockDim.x * VEC) {
-        const int hh = j / DK, c = j - hh * DK;
-        T* dst = out + t * (long)(H * DK) + j;
+    const int QK = q_abs ? DK : P, skip = DK - QK;
+    for (int j = threadIdx.x * VEC; j < H * QK; j += blockDim.x * VEC) {
+        const int hh = j / QK, c = j - hh * QK + skip;
+        T* dst = out + t * (long)(H * QK) + j;
         if constexpr (VEC == 8) {
             if (c < R) {
                 const T* src = q_abs + ((long)hh * T_ + t) * R + c;
@@ -302,7 +303,8 @@ int hyb_latent_rope_store(const void* q_abs, const void* q, long q_row, const vo
     const bool vec = R % 8 == 0 && P % 8 == 0 && (size_t)q_abs % 16 == 0 && (size_t)out % 16 == 0;
 #define LRS(VEC)                                                                                   \
     HYB_DISPATCH(dt, hipLaunchKernelGGL((latent_rope_store_kernel<T, VEC>), dim3(T_),              \
-                                        dim3(threads_for(H * (R + P) / VEC)), lds, s,              \
+                                        dim3(threads_for((q_abs ? H * (R + P) : H * P + R) / VEC)), \
+                                        lds, s,                                                    \
                                         (const T*)q_abs, (const T*)q, q_row, (const T*)dkv, dkv_row, \
                                         (const float*)w, eps, (const int*)positions,               \
                                         (const float*)inv_freq, dims, (T*)k_cache, (T*)v_cache,    \

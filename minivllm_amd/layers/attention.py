@@ -263,6 +263,25 @@ class SinkAttention(nn.Module):
         return out.view(T, self.num_heads * self.v_head_dim)
 
 
+    def forward_latent(self, q_abs: torch.Tensor, q_rot: torch.Tensor) -> torch.Tensor:
+        """The same for a core whose values lie inside the rows of ONE key head, the queries in two
+        parts: q_abs [H,T,R], q_rot [T,H,P] -> [T, H, R] (rows that belong to no sequence of the
+        step are left as they are)."""
+        ctx = get_context()
+        T = q_rot.shape[0]
+        out = torch.empty((T, self.num_heads, self.v_head_dim), dtype=q_rot.dtype, device=q_rot.device)
+        Bd = ctx.num_decode_seqs if ctx.is_prefill else T
+        if ctx.is_prefill and ctx.num_seqs > Bd:
+            ops.latent_attention_prefill(q_abs, q_rot, self.k_cache, ctx.cu_seqlens_q[Bd:],
+                                         ctx.block_tables[Bd:], ctx.positions, self.scale, self.sink, out,
+                                         ctx.max_seqlen_q or None, self.window)
+        if Bd:
+            ops.latent_attention_decode(q_abs[:, :Bd], q_rot[:Bd], self.k_cache, ctx.block_tables[:Bd],
+                                        ctx.context_lens, self.scale, self.sink, out[:Bd],
+                                        ctx.max_context_len or None, self.window)
+        return out
+
+
 class LatentAttention(nn.Module):
     """Attention whose keys and values are expansions of one cached latent per token: key of
     head h = [W_uk_h c | r], value = W_uv_h c, with c the RMS-normed latent (R numbers) and r one
@@ -271,7 +290,8 @@ class LatentAttention(nn.Module):
     scale, and the weighted sum of values is W_uv_h applied to the weighted sum of latents.  So
     this is attention with ONE key/value head whose key row is [c | r] (R + P) and whose value row
     is c (R), run by ``SinkAttention`` (with its window and sink, when asked for), between two
-    batched products per head.  ``up_k`` [H, D, R] and ``up_v`` [H, R, E] are the per-head
+    batched products per head; in bfloat16 on the GPU by a matrix-core kernel of its own that takes
+    the two parts of a query where they are (``SinkAttention.forward_latent``).  ``up_k`` [H, D, R] and ``up_v`` [H, R, E] are the per-head
     expansion matrices, each laid out as the right operand of its product; ``rotation``: a
     ``HalfRotation`` / ``NeighbourRotation`` over the first entries of the P-part.  Only c and r
     are cached, once: the values are read from the key rows (``value_in_key``)."""
@@ -315,11 +335,12 @@ class LatentAttention(nn.Module):
         H, D, R, E = self.num_heads, self.head_dim, self.kv_rank, self.v_head_dim
         q_abs = torch.bmm(q[:, :, :D].transpose(0, 1), self.up_k)                    # [H, T, R]
         rot = self.rotation
-        qf = ops.latent_rope_store(q_abs, q, dkv, self.latent_norm, self.eps, ctx.positions,
+        parts = core.value_in_key and ops.latent_attention_ok(q_abs, core.k_cache, self.rot_dim)
+        qr = ops.latent_rope_store(q_abs, q, dkv, self.latent_norm, self.eps, ctx.positions,
                                    rot.inv_freq, rot.rotary_dim, core.k_cache,
                                    None if core.value_in_key else core.v_cache, ctx.slot_mapping,
-                                   rot.neighbours, rot.mult)
-        o = core(qf, None).view(T, H, R)
+                                   rot.neighbours, rot.mult, assemble=not parts)
+        o = core.forward_latent(q_abs, qr) if parts else core(qr, None).view(T, H, R)
         out = o.new_empty((T, H, E))
         torch.bmm(o.transpose(0, 1), self.up_v, out=out.transpose(0, 1))
         return out

@@ -395,9 +395,31 @@ def row_norm_store(q, k, v, qw, kw, eps, k_cache, v_cache, slot_mapping):
 
 
 def latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims, k_cache, v_cache,
-                      slot_mapping, neighbours=False, mult=1.0):
+                      slot_mapping, neighbours=False, mult=1.0, assemble=True):
+    """``assemble`` False: returns the rotated query parts [T,H,P] alone (for kernels that take the
+    two parts of a query separately)."""
     return _seqmix(q).latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims,
-                                        k_cache, v_cache, slot_mapping, neighbours, mult)
+                                        k_cache, v_cache, slot_mapping, neighbours, mult, assemble)
+
+
+def latent_attention_ok(q_abs, k_cache, rot_dim):
+    """True when attention over these latents has a kernel that takes the parts of a query
+    separately (``latent_attention_prefill`` / ``_decode``)."""
+    return _on_gpu(q_abs) and _hybrid().latent_attention_ok(q_abs, k_cache, rot_dim)
+
+
+def latent_attention_prefill(q_abs, q_rot, k_cache, cu_q, block_tables, positions, scale, sink, out,
+                             max_q=None, window=0):
+    """GPU only (``hip_hybrid``); elsewhere the queries are assembled and ``sink_attention_*`` runs."""
+    return _hybrid().latent_attention_prefill(q_abs, q_rot, k_cache, cu_q, block_tables, positions, scale,
+                                              sink, out, max_q, window)
+
+
+def latent_attention_decode(q_abs, q_rot, k_cache, block_tables, context_lens, scale, sink, out,
+                            max_context_len=None, window=0):
+    """GPU only (``hip_hybrid``)."""
+    return _hybrid().latent_attention_decode(q_abs, q_rot, k_cache, block_tables, context_lens, scale,
+                                             sink, out, max_context_len, window)
 
 
 def xielu(u, ap, aq, out_dtype):

@@ -85,6 +85,12 @@ _hyp = _sig("hyb_hyper_update_norm", _P, _L, _L, _P, _P, _L, _P, _L, _P, _L, _P,
 _cor = _sig("hyb_corrected_route", _P, _P, _P, _P, _L, _I, _I, _I, _I, _F, _I, _P)
 _gtg = _sig("hyb_gelu_tanh_glu", _P, _L, _P, _L, _I, _I, _P)
 
+_lat = _sig("hyb_latent_attention", _P, _L, _L, _P, _L, _L, _P, _P, _I, _I, _P, _P, _P, _P, _P, _L, _L, _P,
+            _F, _I, _I, _I, _I, _I, _I, _I, _P)
+_lat_ok = _lib.hyb_latent_attention_ok
+_lat_ok.argtypes = [_I, _I]
+_lat_ok.restype = _I
+
 _DT = {torch.bfloat16: 0, torch.float32: 2}
 
 
@@ -601,7 +607,7 @@ def row_norm_store(q, k, v, qw, kw, eps, k_cache, v_cache, slot_mapping):
 
 
 def latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims, k_cache, v_cache,
-                      slot_mapping, neighbours=False, mult=1.0):
+                      slot_mapping, neighbours=False, mult=1.0, assemble=True):
     H, T, R = q_abs.shape
     P = dkv.shape[1] - R
     D = q.shape[2] - P
@@ -612,12 +618,70 @@ def latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims, k_ca
         assert k_cache.is_contiguous() and k_cache.dtype == q.dtype and k_cache.shape[2:] == (1, R + P)
         if v_cache is not None:          # None: the values are the leading part of the key rows
             assert v_cache.is_contiguous() and v_cache.shape[2:] == (1, R)
-    out = torch.empty((T, H, R + P), dtype=q.dtype, device=q.device)
-    _check(_lrs(q_abs.data_ptr(), q.data_ptr(), _rows(q), dkv.data_ptr(), _rows(dkv),
+    out = torch.empty((T, H, R + P if assemble else P), dtype=q.dtype, device=q.device)
+    _check(_lrs(q_abs.data_ptr() if assemble else None, q.data_ptr(), _rows(q), dkv.data_ptr(), _rows(dkv),
                 _f32(w).data_ptr(), eps, _i32(positions).data_ptr(), _f32(inv_freq).data_ptr(),
                 int(rot_dims), _ptr(k_cache), _ptr(v_cache), _ptr(_i32(slot_mapping)), out.data_ptr(),
                 T, H, D, P, R, int(neighbours), float(mult), _dt(q), _stream()), "latent_rope_store")
     return out
+
+
+# ------------------------------------------------------------------ attention over shared latents
+def latent_attention_ok(q_abs, k_cache, rot_dim: int) -> bool:
+    """True when the matrix-core kernel has an instance: bfloat16, latents of up to 512 numbers,
+    sizes in whole runs of eight."""
+    return bool(q_abs.dtype == torch.bfloat16 and k_cache is not None and k_cache.dtype == torch.bfloat16
+                and k_cache.is_contiguous() and rot_dim > 0 and _lat_ok(q_abs.shape[2], rot_dim))
+
+
+def latent_splits(batch: int, heads: int, latent: int, max_context_len, window: int = 0) -> int:
+    """Workgroups per sequence and 32 query rows for single next tokens: one per compute unit for
+    latents above 256 numbers (a workgroup fills its LDS and registers), several below, each with at
+    least 128 keys of the longest context."""
+    tiles = batch * -(-heads // 32) if heads <= 64 else batch * -(-heads // 128)
+    want = -(-(256 if latent > 256 else 768) // max(tiles, 1))
+    seen = min(int(max_context_len), window + 31) if window and max_context_len else max_context_len
+    room = max(1, (int(seen) + 127) // 128) if seen else 8
+    return max(1, min(16, want, room))
+
+
+def _latent(q_abs, q_rot, k_cache, tables, cu_q, positions, lens, scale, sink, out, nseq, max_q, window, splits):
+    H, T, R = q_abs.shape
+    P = q_rot.shape[2]
+    assert q_abs.stride(2) == 1 and q_rot.stride(2) == 1 and q_rot.shape[:2] == (T, H)
+    assert out.shape == (T, H, R) and out.stride(2) == 1 and k_cache.is_contiguous() \
+        and k_cache.shape[2:] == (1, R + P) and q_abs.dtype == q_rot.dtype == out.dtype == k_cache.dtype
+    assert tables.dtype == torch.int32 and tables.stride(1) == 1 and tables.shape[0] >= nseq
+    ws = None
+    if splits > 1:
+        assert out.is_contiguous()
+        ws = torch.empty((nseq * H * splits * (R + 2),), dtype=torch.float32, device=out.device)
+    _check(_lat(q_abs.data_ptr(), q_abs.stride(1), q_abs.stride(0), q_rot.data_ptr(), q_rot.stride(0),
+                q_rot.stride(1), k_cache.data_ptr(), tables.data_ptr(), tables.stride(0), k_cache.shape[1],
+                _ptr(cu_q), _ptr(positions), _ptr(lens), _ptr(_f32(sink)) if sink is not None else None,
+                out.data_ptr(), out.stride(0), out.stride(1), _ptr(ws), float(scale), nseq, int(max_q), H, R,
+                P, int(window), int(splits), _stream()), "latent_attention")
+    return out
+
+
+def latent_attention_prefill(q_abs, q_rot, k_cache, cu_q, block_tables, positions, scale, sink, out,
+                             max_q, window=0):
+    """Prompt portions: ``q_abs`` [H, T, R] and ``q_rot`` [T, H, P] are the two parts of the queries,
+    sequence b owns rows cu_q[b] .. cu_q[b+1] (absolute rows) and block table row b; ``max_q``: the
+    longest portion (a host integer)."""
+    nseq = cu_q.shape[0] - 1
+    if max_q is None:
+        max_q = int((cu_q[1:] - cu_q[:-1]).max())
+    return _latent(q_abs, q_rot, k_cache, block_tables, _i32c(cu_q), _i32(positions), None, scale, sink, out,
+                   nseq, max_q, window, 1)
+
+
+def latent_attention_decode(q_abs, q_rot, k_cache, block_tables, context_lens, scale, sink, out,
+                            max_context_len=None, window=0):
+    """Single next tokens: row b is sequence b with ``context_lens[b]`` keys."""
+    B, H, R = out.shape
+    return _latent(q_abs, q_rot, k_cache, block_tables, None, None, _i32c(context_lens), scale, sink, out,
+                   B, 1, window, latent_splits(B, H, R, max_context_len, window))
 
 
 def xielu(u, ap, aq, out_dtype):

@@ -540,7 +540,7 @@ def _rotate(x, positions, inv_freq, dims, neighbours=False, mult=1.0):
 
 
 def latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims, k_cache, v_cache,
-                      slot_mapping, neighbours=False, mult=1.0):
+                      slot_mapping, neighbours=False, mult=1.0, assemble=True):
     """Assembles the queries and cache rows of attention over a shared latent.  ``q_abs`` [H,T,R]:
     the heads' unrotated query parts carried into the latent's coordinates; ``q`` [T,H,D+P] whose
     last P entries per head are the part to rotate; ``dkv`` [T,R+P]: the raw latent and one key
@@ -548,14 +548,15 @@ def latent_rope_store(q_abs, q, dkv, w, eps, positions, inv_freq, rot_dims, k_ca
     head of R + P), V cache row = the normed latent (R; ``v_cache`` None: not written, the reader
     takes the leading R entries of the key rows).  Returns the queries [T,H,R+P] =
     [q_abs | rotated part].  The rotation turns the first ``rot_dims`` of the P entries in
-    half-split pairs, or in pairs of ``neighbours``, cos and sin both times ``mult``."""
+    half-split pairs, or in pairs of ``neighbours``, cos and sin both times ``mult``.  ``assemble``
+    False: the rotated query parts [T,H,P] alone are returned."""
     H, T, R = q_abs.shape
     P = dkv.shape[1] - R
     D = q.shape[2] - P
     c = rms_norm_rows(dkv[:, :R], w, eps, torch.float32)
     kr = _rotate(dkv[:, R:].float(), positions, inv_freq, rot_dims, neighbours, mult)
     qr = _rotate(q[:, :, D:].float(), positions, inv_freq, rot_dims, neighbours, mult)
-    out = torch.cat([q_abs.transpose(0, 1).float(), qr], -1).to(q.dtype)
+    out = (torch.cat([q_abs.transpose(0, 1).float(), qr], -1) if assemble else qr).to(q.dtype)
     if k_cache is not None and slot_mapping is not None:
         _scatter_rows(k_cache, torch.cat([c, kr], -1)[:, None, :], slot_mapping)
         if v_cache is not None:          # None: the values are the leading part of the key rows

@@ -115,3 +115,83 @@ def test_latent_queries_and_cache_rows(dt, H, D, P, R, dims, cls):
         res[name] = (out.cpu().float(), cache.cpu().float())
     for a, b in zip(res["gpu"], res["cpu"]):
         torch.testing.assert_close(a, b, **(tol(dt) if dt == torch.bfloat16 else dict(rtol=1e-3, atol=1e-3)))
+
+
+LATENT_CASES = [
+    # H, R, P, block size, window: one per instance and form of the kernel, padded sizes, pages that
+    # are shorter than a key tile or no divisor of it, more heads than one tile of query rows
+    (16, 64, 32, 64, 0), (6, 96, 32, 32, 0), (8, 128, 32, 64, 0), (16, 128, 128, 256, 70), (3, 40, 24, 8, 0),
+    (16, 256, 64, 64, 0), (5, 200, 96, 16, 33), (16, 512, 64, 64, 0), (7, 384, 128, 12, 0), (48, 128, 64, 64, 0),
+    (80, 512, 64, 32, 0), (1, 8, 8, 4, 5), (128, 256, 128, 64, 100)]
+
+
+@pytest.mark.parametrize("H,R,P,bs,window", LATENT_CASES)
+@pytest.mark.parametrize("with_sink", [False, True])
+def test_latent_attention(H, R, P, bs, window, with_sink):
+    """The matrix-core kernel against the plain attention on assembled queries: portions of several
+    sequences (one shorter than a tile, one that starts late, one of two tokens), then their last
+    rows as single tokens with every number of context splits.  One key of the longest sequence is
+    made to stand out for every query."""
+    from minivllm_amd.ops import torch_seqmix
+    torch.manual_seed(R + H)
+    dt = torch.bfloat16
+    lens, qlens = [150, 37, 290, 64], [150, 30, 2, 1]
+    B, D = len(lens), R + P
+    pages = [-(-n // bs) for n in lens]
+    perm = torch.randperm(sum(pages) + 2).tolist()
+    tables, at = torch.zeros(B, max(pages), dtype=torch.int32), 0
+    for b, n in enumerate(pages):
+        tables[b, :n] = torch.tensor(perm[at:at + n], dtype=torch.int32)
+        at += n
+    cache = torch.randn(sum(pages) + 2, bs, 1, D).to(dt)
+    T = sum(qlens)
+    q_abs, q_rot = torch.randn(H, T, R).to(dt), torch.randn(T, H, P).to(dt)
+    far = 3                                                          # (behind every window used here)
+    cache[int(tables[2, far // bs]), far % bs, 0] = torch.cat([q_abs[0, 181], q_rot[181, 0]]) * 2.0
+    sink = 2.0 * torch.randn(H) if with_sink else None
+    scale = 1.5 * D ** -0.5
+    cu_q = torch.tensor([0, 150, 180, 182, 183], dtype=torch.int32)
+    cu_k = torch.tensor([0] + torch.tensor(lens).cumsum(0).tolist(), dtype=torch.int32)
+    pos = torch.cat([torch.arange(n - m, n) for n, m in zip(lens, qlens)]).to(torch.int32)
+    q = torch.cat([q_abs.transpose(0, 1), q_rot], -1)
+    v = cache[..., :R]
+    want = torch.zeros(T, H, R)
+    torch_seqmix.sink_attention_prefill(q, cache, v, cu_q, cu_k, tables, scale, sink, None, want, window)
+    assert hk.latent_attention_ok(q_abs.cuda(), cache.cuda(), P)
+    gq, gr, gc, gs, gt = q_abs.cuda(), q_rot.cuda(), cache.cuda(), up(sink), tables.cuda()
+    got = torch.full((T, H, R), float("nan"), dtype=dt, device="cuda")
+    hk.latent_attention_prefill(gq, gr, gc, cu_q.cuda(), gt, pos.cuda(), scale, gs, got, max(qlens), window)
+    torch.testing.assert_close(got.cpu().float(), want, rtol=1e-2, atol=1e-2)
+    # the sequences behind the first alone, as a step with riders slices them
+    part = torch.full_like(got, float("nan"))
+    hk.latent_attention_prefill(gq, gr, gc, cu_q.cuda()[1:], gt[1:], pos.cuda(), scale, gs, part, max(qlens), window)
+    assert torch.equal(part[150:], got[150:]) and bool(torch.isnan(part[:150]).all())
+    last = (cu_q[1:] - 1).long()
+    ctx = torch.tensor(lens + [0], dtype=torch.int32)                # an unused row of a padded batch
+    last5 = torch.cat([last, torch.zeros(1, dtype=torch.long)])
+    t5 = torch.cat([tables, torch.zeros_like(tables[:1])])
+    for splits in (1, 2, 3, 8):
+        dec = torch.full((5, H, R), float("nan"), dtype=dt, device="cuda")
+        hk._latent(gq[:, last5].contiguous(), gr[last5].contiguous(), gc, t5.cuda(), None, None, ctx.cuda(), scale, gs,
+                   dec, 5, 1, window, splits)
+        torch.testing.assert_close(dec[:4].cpu().float(), want[last], rtol=1e-2, atol=1e-2)
+        assert bool(torch.isnan(dec[4]).all())                       # left as it was
+
+
+def test_latent_weights_keep_more_than_sixteen_bits():
+    """Two keys with almost equal scores and opposite values: with weights rounded to bfloat16 the
+    difference is lost altogether."""
+    R, P, H = 64, 8, 2
+    cache = torch.zeros(1, 64, 1, R + P, dtype=torch.bfloat16)
+    cache[0, 1, 0, R] = -0.0015                                      # scores, carried by the key part alone
+    cache[0, 0, 0, 0], cache[0, 1, 0, 0] = 100.0, -100.0
+    q_abs = torch.zeros(H, 1, R, dtype=torch.bfloat16)
+    q_rot = torch.zeros(1, H, P, dtype=torch.bfloat16)
+    q_rot[..., 0] = 1.0
+    p = torch.exp(cache[0, :2, 0, R].double())
+    want = float(100.0 * (p[0] - p[1]) / p.sum())
+    out = torch.zeros(1, H, R, dtype=torch.bfloat16, device="cuda")
+    hk._latent(q_abs.cuda(), q_rot.cuda(), cache.cuda(), torch.zeros(1, 1, dtype=torch.int32, device="cuda"), None, None,
+               torch.tensor([2], dtype=torch.int32, device="cuda"), 1.0, None, out, 1, 1, 0, 1)
+    assert want > 0.07 and float(p[1].to(torch.bfloat16)) == 1.0
+    assert abs(float(out[0, 0, 0]) - want) < 0.02 * want
