@@ -107,31 +107,32 @@ hyper_kernel(const float* xi, long xi_t, long xi_s, float* xo, const T* __restri
     store_vec<T, VEC>(h + t * (long)W + c, u);
 }
 
-// sums of 8 * TOK values over a wave, the results spread over the lanes: every exchange halves the
-// number of values a lane still carries.  Returns the total of value index `slot(lane)`.
-template <int N>
-__device__ __forceinline__ float scatter_sum(float* v, int lane, int& slot) {
-    slot = 0;
-    int o = 32;
+// sums of N values over a wave, the results spread over the lanes: every exchange halves the number
+// of values a lane still carries (N a power of two).  A lane returns the total of value `slot`.
+template <int N, int O = kWave / 2>
+__device__ __forceinline__ float scatter_sum(float (&v)[N], int lane, int& slot) {
+    if constexpr (N == 1) {
+        float s = v[0];
 #pragma unroll
-    for (int n = N; n > 1; n >>= 1, o >>= 1) {
-        const bool up = lane & o;
+        for (int o = O; o > 0; o >>= 1) s += __shfl_xor(s, o, kWave);
+        return s;
+    } else {
+        const bool up = lane & O;
+        float half[N / 2];
 #pragma unroll
-        for (int i = 0; i < n / 2; ++i) {
-            const float send = up ? v[i] : v[i + n / 2];
-            const float keep = up ? v[i + n / 2] : v[i];
-            v[i] = keep + __shfl_xor(send, o, kWave);
+        for (int i = 0; i < N / 2; ++i) {
+            const float send = up ? v[i] : v[i + N / 2];
+            const float keep = up ? v[i + N / 2] : v[i];
+            half[i] = keep + __shfl_xor(send, O, kWave);
         }
         slot = slot * 2 + (up ? 1 : 0);
+        return scatter_sum<N / 2, O / 2>(half, lane, slot);
     }
-    float s = v[0];
-    for (; o > 0; o >>= 1) s += __shfl_xor(s, o, kWave);
-    return s;
 }
 
 // One workgroup (4 waves) per TOK token rows: the rows of the router matrix are read once per
 // workgroup, eight at a time; then wave k softmaxes and chooses for token k.  z: [TOK][NR] in LDS.
-template <typename T, int TOK>
+template <typename T, int TOK, int VEC>
 __global__ void __launch_bounds__(256)
 corrected_route_kernel(const T* __restrict__ h, const float* __restrict__ wr,
                        const float* __restrict__ corr, float* __restrict__ dense, long T_, int W,
@@ -146,19 +147,21 @@ corrected_route_kernel(const T* __restrict__ h, const float* __restrict__ wr,
         float acc[8 * TOK];
 #pragma unroll
         for (int j = 0; j < 8 * TOK; ++j) acc[j] = 0.f;
-#pragma unroll 2
-        for (int c = threadIdx.x; c < W; c += 256) {
-            float hv[TOK];
+        for (int c = threadIdx.x * VEC; c < W; c += 256 * VEC) {
+            float hv[TOK][VEC];
 #pragma unroll
-            for (int k = 0; k < TOK; ++k) hv[k] = t0 + k < T_ ? ld(h + (t0 + k) * W + c) : 0.f;
+            for (int k = 0; k < TOK; ++k) load_vec<T, VEC>(h + min(t0 + k, T_ - 1) * W + c, hv[k]);
 #pragma unroll
             for (int j = 0; j < 8; ++j) {
-                const float wv = e0 + j < NR ? wr[(long)(e0 + j) * W + c] : 0.f;
+                float wv[VEC];
+                load_vec<float, VEC>(wr + (long)min(e0 + j, NR - 1) * W + c, wv);
 #pragma unroll
-                for (int k = 0; k < TOK; ++k) acc[k * 8 + j] += hv[k] * wv;
+                for (int k = 0; k < TOK; ++k)
+#pragma unroll
+                    for (int i = 0; i < VEC; ++i) acc[k * 8 + j] += hv[k][i] * wv[i];
             }
         }
-        int slot;
+        int slot = 0;
         const float s = scatter_sum<8 * TOK>(acc, lane, slot);
         if ((lane & (kWave / (8 * TOK) - 1)) == 0) red[wave * 8 * TOK + slot] = s;
         __syncthreads();
@@ -297,14 +300,17 @@ int hyb_corrected_route(const void* h, const void* wr, const void* corr, void* d
                         int NE, int NR, int top, float scale, int dt, hipStream_t s) {
     if (T_ <= 0) return 0;
     if (NE < 0 || NR < NE || NR < 1 || top < 1 || top > NR || NR > 1536) return 1;
-#define ROUTE(TOK)                                                                                 \
-    HYB_DISPATCH(dt, hipLaunchKernelGGL((corrected_route_kernel<T, TOK>),                           \
+    const bool vec = W % 4 == 0 && ((size_t)h | (size_t)wr) % 16 == 0;
+#define ROUTE_VEC(TOK, VEC)                                                                        \
+    HYB_DISPATCH(dt, hipLaunchKernelGGL((corrected_route_kernel<T, TOK, VEC>),                      \
                                         dim3((unsigned)((T_ + TOK - 1) / TOK)), dim3(256),         \
                                         (2 * TOK * NR + 32 * TOK) * sizeof(float), s, (const T*)h, \
                                         (const float*)wr, (const float*)corr, (float*)dense, T_, W, \
                                         NE, NR, top, scale))
+#define ROUTE(TOK) do { if (vec) ROUTE_VEC(TOK, 4); else ROUTE_VEC(TOK, 1); } while (0)
     if (T_ >= 2048) ROUTE(4); else ROUTE(1);
 #undef ROUTE
+#undef ROUTE_VEC
     return HYB_LAUNCH_OK();
 }
 

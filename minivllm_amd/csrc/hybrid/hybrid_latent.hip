@@ -25,7 +25,7 @@
 // take the left / right half of the value columns, waves 0, 2 / 1, 3 the even / odd key tiles; the
 // two halves of the keys meet in LDS at the end, the context may be split over workgroups too (fp32
 // partials in a workspace, folded by the merge kernel).  Key tiles are double-buffered in LDS by
-// direct global -> LDS loads; the next one is requested between the softmax and the P V products.
+// direct global -> LDS loads, requested a stage ahead.
 //
 // EP: value columns the accumulators hold (R <= EP, a multiple of 32); DP: key columns of the LDS
 // image (R + P <= DP, a multiple of 64).  The image is XOR-swizzled in 16-byte chunks so that both
@@ -157,6 +157,15 @@ latent_attention_kernel(LatentArgs a) {
         s_off[i] = row * D * 2 + ch * 16;
     }
     const bool uniform_rows = (a.block_size & 31) == 0;             // a tile's rows are consecutive
+    // block ids of a stage's tiles, through the scalar unit (the table is read-only here) and a stage
+    // early: a vector load would be waited for together with everything else in flight
+    int ids[KW];
+    auto fetch_ids = [&](int t0) {
+        typedef const __attribute__((address_space(4))) int* const_int_p;
+#pragma unroll
+        for (int k = 0; k < KW; ++k)
+            ids[k] = *(const_int_p)(uintptr_t)(table + min((t0 + k) * 32, n_keys - 1) / a.block_size);
+    };
     auto stage = [&](int t0, int buf) {
 #pragma unroll
         for (int k = 0; k < KW; ++k) {
@@ -164,8 +173,7 @@ latent_attention_kernel(LatentArgs a) {
             if (key0 >= n_keys) continue;
             char* dst = smem + (buf * KW + k) * TILE + wave * 1024;
             if (uniform_rows) {
-                const int blk = __builtin_amdgcn_readfirstlane(table[key0 / a.block_size]);
-                const uint16_t* src = a.cache + ((long)blk * a.block_size + key0 % a.block_size) * D;
+                const uint16_t* src = a.cache + ((long)ids[k] * a.block_size + key0 % a.block_size) * D;
                 // rows behind the context are out of the buffer's range and read as zeros
                 const int bytes = min(32, n_keys - key0) * D * 2;
                 const __amdgpu_buffer_rsrc_t rsrc = __builtin_amdgcn_make_buffer_rsrc(
@@ -213,13 +221,21 @@ latent_attention_kernel(LatentArgs a) {
     float m_run = NO_SINK_MAX, l_run = 0.f;         // in log2 units of the scaled scores
     const float sc = a.scale * LOG2E;
 
-    if (t_begin < t_end) stage(t_begin, 0);
+    if (t_begin < t_end) {
+        fetch_ids(t_begin);
+        stage(t_begin, 0);
+        if (t_begin + KW < t_end) fetch_ids(t_begin + KW);
+    }
     __syncthreads();
     for (int t = t_begin, buf = 0; t < t_end; t += KW, buf ^= 1) {
         const int key0 = (t + kw) * 32;
         const bool live = wave_live && t + kw < t_end && key0 <= w_last &&
                           (a.window <= 0 || key0 + 31 > w_first - a.window);       // (uniform per wave)
         bf16x8 p_hi[2], p_lo[2];
+        if (t + KW < t_end) {                           // lands behind this tile's products
+            stage(t + KW, buf ^ 1);
+            if (t + 2 * KW < t_end) fetch_ids(t + 2 * KW);
+        }
         if (live) {
             f32x16 s_acc;
 #pragma unroll
@@ -255,17 +271,19 @@ latent_attention_kernel(LatentArgs a) {
             // lane: query row l32, keys key0 + (e & 3) + 8 (e >> 2) + 4 half
             const bool all_seen = key0 + 31 <= w_first && (a.window <= 0 || w_last - key0 < a.window);
             const int oldest = a.window > 0 ? qpos - a.window : -1;
+            if (!all_seen) {                             // (one uniform branch, not one per score)
+#pragma unroll
+                for (int e = 0; e < 16; ++e) {
+                    const int key = key0 + (e & 3) + 8 * (e >> 2) + 4 * half;
+                    s_acc[e] = ((key > qpos) | (key <= oldest)) ? -INFINITY : s_acc[e] * sc;
+                }
+            } else {
+#pragma unroll
+                for (int e = 0; e < 16; ++e) s_acc[e] *= sc;
+            }
             float mt = -INFINITY;
 #pragma unroll
-            for (int e = 0; e < 16; ++e) {
-                float v = s_acc[e] * sc;
-                if (!all_seen) {
-                    const int key = key0 + (e & 3) + 8 * (e >> 2) + 4 * half;
-                    v = ((key > qpos) | (key <= oldest)) ? -INFINITY : v;
-                }
-                s_acc[e] = v;
-                mt = fmaxf(mt, v);
-            }
+            for (int e = 0; e < 16; ++e) mt = fmaxf(mt, s_acc[e]);
             mt = fmaxf(mt, __shfl_xor(mt, 32, kWave));
             // the reference of the exponentials only moves when some row outgrows it by RESCALE
             if (!__all(mt - m_run <= RESCALE)) {
@@ -291,7 +309,6 @@ latent_attention_kernel(LatentArgs a) {
                 p_lo[s] = __builtin_bit_cast(bf16x8, lo);
             }
         }
-        if (t + KW < t_end) stage(t + KW, buf ^ 1);     // lands behind the products below
         if (live) {
             // transposed reads as inline asm: through the builtin the compiler would wait for the
             // stage's loads in flight ahead of the first one.  Step i (value block i / 2, keys 16
