@@ -4,7 +4,7 @@
 //   rms_norm_rows       rows of an activation tensor / rms * w            (a latent's norm)
 //   row_norm_store      q and k RMS-normed over their WHOLE projection (all heads at once), or
 //                       left as they are; k and v written to their cache slot
-//   latent_rope_store   latent norm + half-split rotation + query assembly + cache write
+//   latent_rope_store   latent norm + rotation (either pair layout) + query assembly + cache write
 //   xielu               the piecewise quadratic / exponential activation
 //   gated_group_norm    (o + skip x) silu(z), RMS norm in equal parts, weight
 //   sigmoid_gate        o * sigmoid(g) element by element, gathering a head-major o

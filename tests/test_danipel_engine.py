@@ -509,3 +509,15 @@ def test_engine_refuses_what_the_kernels_do_not_take(tmp_path):
     bad["layers"][0]["type"] = "latent_attention_3"
     with pytest.raises(ValueError, match="latent_attention_3"):
         cfg(bad)
+
+
+def test_benchmark_configuration_parses_and_validates():
+    import types
+    sys.path.insert(0, ROOT)
+    import bench
+    for size in ("w1024", "w2048"):
+        mc = bench.danipel_model(size)
+        mc.validate_engine(types.SimpleNamespace(tp_degree=1))
+        kinds = [L.type for L in mc.layers]
+        assert len(kinds) == 8 and kinds.count("latent_attention") == 4 and mc.streams == 2
+        assert [L.mlp["kind"] for L in mc.layers] == ["dense"] + ["moe"] * 7
