@@ -19,6 +19,13 @@ class GeluTanhAndMul(nn.Module):
         return ops.gelu_tanh_glu(x, x.dtype)
 
 
+class ReluSquared(nn.Module):
+    """``max(x, 0)^2``, fp32 arithmetic."""
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return ops.relu_squared(x, x.dtype)
+
+
 class XIELU(nn.Module):
     """xIELU with two learned numbers p, q: ``softplus(p) z^2 + z/2`` for z > 0 and
     ``(1/2 + softplus(q)) (e^z - 1 - z) + z/2`` otherwise.  The two coefficients are worked out

@@ -25,6 +25,7 @@ import torch
 import torch.nn as nn
 
 from minivllm_amd import ops
+from minivllm_amd.layers.state_space import StateSlots
 from minivllm_amd.utils.context import get_context
 
 
@@ -170,7 +171,9 @@ class SinkAttention(nn.Module):
     Options, each a constructor argument: ``sink=False`` - an ordinary softmax (no extra term);
     ``window`` > 0 - a query at position i sees key j <= i only when i - j < window or
     j < keep_first (the first tokens stay visible at their true positions); ``distance_slopes``
-    [H] - slope_h * (i - j) is taken off the score of key j; ``value_in_key`` - a token's value is
+    [H] - slope_h * (i - j) is taken off the score of key j; ``chunk`` > 0 - a query sees only keys
+    of its own run of ``chunk`` positions (counted from position 0 of the sequence);
+    ``value_in_key`` - a token's value is
     the leading ``v_head_dim`` entries of its key row, so the engine allocates no V cache and
     ``v_cache`` is a view into ``k_cache``; ``head_temps`` - a learned multiplier per query head
     on the scaled score (``temps`` [H] fp32); ``softcap`` > 0 - score <- softcap tanh(score /
@@ -184,8 +187,11 @@ class SinkAttention(nn.Module):
     def __init__(self, num_heads: int, num_kv_heads: int, head_dim: int, v_head_dim: int,
                  scale: float, sink: bool = True, window: int = 0, keep_first: int = 0,
                  distance_slopes: Optional[torch.Tensor] = None, value_in_key: bool = False,
-                 head_temps: bool = False, softcap: float = 0.0, pool: int = 0):
+                 head_temps: bool = False, softcap: float = 0.0, pool: int = 0, chunk: int = 0):
         super().__init__()
+        if chunk and (keep_first or pool):
+            raise ValueError("chunks combine with neither kept first tokens nor pooled blocks")
+        self.chunk = int(chunk)
         if pool and (not window or keep_first or value_in_key or distance_slopes is not None):
             raise ValueError("pooled blocks need a window and combine with neither kept first "
                              "tokens, a distance penalty nor values inside the key rows")
@@ -243,6 +249,8 @@ class SinkAttention(nn.Module):
         if self.temps is not None or self.softcap or self.pool:
             opt.update(temps=self.temps, softcap=self.softcap, pool=self.pool, k_pool=self.k_pool,
                        v_pool=self.v_pool)
+        if self.chunk:
+            opt.update(chunk=self.chunk)
         if not ctx.is_prefill:
             ops.sink_attention_decode(q, *a, ctx.block_tables, ctx.context_lens, self.scale,
                                       self.sink, gate, out, ctx.max_context_len or None, **opt)
@@ -280,6 +288,39 @@ class SinkAttention(nn.Module):
                                         ctx.context_lens, self.scale, self.sink, out[:Bd],
                                         ctx.max_context_len or None, self.window)
         return out
+
+
+class FilteredHeads(nn.Module):
+    """What stands between a fused q / k / v projection and attention in models that filter their
+    heads: a causal filter over time of ``taps`` taps on every projected channel (no bias, no
+    activation), then an RMS norm per q head and per k head with one weight of ``head_dim`` numbers
+    each, then the cache write.  ``forward`` returns the queries.  A pass of the layer keeps the
+    last taps - 1 projected rows per sequence (``StateSlots``)."""
+
+    def __init__(self, num_heads: int, num_kv_heads: int, head_dim: int, v_head_dim: int, taps: int,
+                 eps: float, passes: int = 1):
+        super().__init__()
+        H, G, D, E = num_heads, num_kv_heads, head_dim, v_head_dim
+        self.sizes, self.taps, self.eps = (H, G, D, E), int(taps), eps
+        self.channels = H * D + G * D + G * E
+        f32 = dict(dtype=torch.float32)
+        # taps of the q, k and v channels stacked in that order (last column = current token)
+        self.conv_weight = nn.Parameter(torch.zeros(self.channels, self.taps, **f32), requires_grad=False)
+        self.q_norm = nn.Parameter(torch.ones(D, **f32), requires_grad=False)
+        self.k_norm = nn.Parameter(torch.ones(D, **f32), requires_grad=False)
+        spec = [("conv_state", (self.taps - 1, self.channels))] if self.taps > 1 else []
+        self.slots = [StateSlots(spec) for _ in range(passes)]
+
+    def forward(self, proj: torch.Tensor, core: SinkAttention, which: int = 0) -> torch.Tensor:
+        """proj [T, >= channels] (q, k, v side by side) -> q [T, H, D]; k and v of every row are in
+        ``core``'s cache afterwards."""
+        ctx = get_context()
+        pre = ctx.is_prefill
+        return ops.conv_norm_store(proj, self.sizes, self.conv_weight,
+                                   self.slots[which].conv_state if self.taps > 1 else None, self.q_norm,
+                                   self.k_norm, self.eps, core.k_cache, core.v_cache, ctx.slot_mapping,
+                                   ctx.cu_seqlens_q if pre else None, ctx.positions, ctx.state_slots,
+                                   row_seq=ctx.row_seq if pre else None)
 
 
 class LatentAttention(nn.Module):

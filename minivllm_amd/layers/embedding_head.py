@@ -118,3 +118,63 @@ class SinusoidalEmbedding(nn.Module):
 
     def forward(self, ids: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
         return ops.embed_sinusoid(ids, positions, self.weight, self.inv_freq)
+
+
+class ScaledTiedHead(nn.Module):
+    """Final RMS norm, then the embedding table itself as the output projection, times a constant.
+    The constant is folded into the norm's fp32 gain (``gain`` = weight * logit_scale), so the
+    logits are rounded once; ``offset``: the stored norm weight is an offset from this number.  Applied to the rows a step wants (each sequence's last row, or the
+    context's ``logit_rows``)."""
+
+    def __init__(self, embedding: nn.Embedding, eps: float, logit_scale: float = 1.0, offset: float = 0.0):
+        super().__init__()
+        self.table = [embedding]                     # not a submodule: the weight is the model's
+        self.eps, self.logit_scale, self.offset = eps, float(logit_scale), float(offset)
+        W = embedding.weight.shape[1]
+        self.weight_norm = nn.Parameter(torch.ones(W, dtype=torch.float32), requires_grad=False)
+        self.gain = nn.Parameter(torch.ones(W, dtype=torch.float32), requires_grad=False)
+        self.num_embeddings = embedding.weight.shape[0]
+        self.vocab_start = 0
+
+    @property
+    def weight(self) -> torch.Tensor:
+        return self.table[0].weight
+
+    @torch.no_grad()
+    def load_norm(self, t: torch.Tensor) -> None:
+        self.weight_norm.copy_(t)
+        self.gain.copy_((self.weight_norm + self.offset) * self.logit_scale)
+
+    def select_last(self, hidden: torch.Tensor) -> torch.Tensor:
+        ctx = get_context()
+        if ctx.logit_rows is not None:
+            return hidden.index_select(0, ctx.logit_rows.long())
+        if ctx.is_prefill and ctx.cu_seqlens_q is not None:
+            return hidden.index_select(0, (ctx.cu_seqlens_q[1:] - 1).long())
+        return hidden
+
+    def local_logits(self, hidden: torch.Tensor) -> torch.Tensor:
+        rows = self.select_last(hidden)
+        w = self.weight
+        return F.linear(ops.group_rms_norm(rows, self.gain, 1, self.eps, w.dtype), w)
+
+    def forward(self, hidden: torch.Tensor) -> torch.Tensor:
+        return self.local_logits(hidden)
+
+
+class LayerTokenInput(nn.Module):
+    """A token's own contribution to ONE layer: y = P (gelu_tanh(G x) * e) with e the layer's run of
+    ``dim`` numbers of a token's row in a table that all layers share.  x comes in rounded to the
+    activation type; y goes out before its norm, which belongs to the stream update
+    (``ops.post_norm_residual``).  ``offset``: where the layer's run starts in a row."""
+
+    def __init__(self, width: int, dim: int, offset: int):
+        super().__init__()
+        self.dim, self.offset = int(dim), int(offset)
+        self.gate = nn.Parameter(torch.zeros(dim, width), requires_grad=False)
+        self.proj = nn.Parameter(torch.zeros(width, dim), requires_grad=False)
+        self.norm_weight = nn.Parameter(torch.ones(width, dtype=torch.float32), requires_grad=False)
+
+    def forward(self, x: torch.Tensor, ids: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
+        g = ops.token_gate(F.linear(x, self.gate), ids, table, self.offset, x.dtype)
+        return F.linear(g, self.proj)

@@ -1,7 +1,7 @@
 """Linear-attention mixers with a per-sequence matrix state S [D, E] per head, fp32, carried from
 token to token in the engine's state slots (a sequence that starts at position 0 starts from
-zeros whatever its slot held).  Both take the raw projections of a step's rows and leave the
-activation of their gates, which is fp32 work, to the scan kernel.
+zeros whatever its slot held).  All leave the activation of their gates and decays, which is fp32
+work, to the scan kernel; the first two take the raw projections of a step's rows.
 
 ``MatrixLSTM``: exponential input gate and sigmoid forget gate in the log domain, both soft-capped,
 stabilised by a running maximum m that starts at 0:
@@ -20,15 +20,25 @@ Short-Term Memory", Beck et al., 2024.)
 
 q scaled by D^-1/2, each head's o RMS-normalised with a weight shared by the heads, times silu of
 a gate projection.
+
+``TokenShiftWKV``: RWKV-style time mixing.  With d = h_(t-1) - h_t (h_(-1) = 0) the receptance r,
+key k, value v, gate g and decay w read h + mu d, each with its own vector mu,
+
+    w = exp(-exp(W_2 tanh(W_1 .) + w_0));   o = (S + diag(u) k v^T)^T r;   S <- diag(w) S + k v^T
+
+(the bonus u weighs the current token alone), each head's o divided by its root mean square, times
+a weight over all heads' outputs, times silu of the gate.
 """
 from __future__ import annotations
 
-from typing import Optional
+from typing import List, Optional
 
 import torch
 import torch.nn as nn
+import torch.nn.functional as F
 
 from minivllm_amd import ops
+from minivllm_amd.layers.state_space import StateSlots
 from minivllm_amd.utils.context import get_context
 
 
@@ -107,3 +117,43 @@ class GatedLinearAttention(nn.Module):
                          self.decay_bias, self.tau, self.state, *_layout(get_context()))
         return ops.gated_head_norm(o, self.norm_weight, gate, self.eps, out_dtype,
                                    "silu").view(T, H * E)
+
+
+class TokenShiftWKV(nn.Module):
+    """The whole mixer up to its output projection; ``forward`` takes the mixer's input.  The four
+    projections of different inputs are ONE batched product: ``proj`` [4, W, H*D] holds W_r^T, W_k^T,
+    W_v^T, W_g^T as right operands.  A pass keeps the matrix state and the previous token's h per
+    sequence (``StateSlots``); a layer that runs several times per token has one per pass."""
+
+    MIXES = ("r", "k", "v", "g", "w")
+
+    def __init__(self, width: int, num_heads: int, head_dim: int, eps: float, passes: int = 1):
+        super().__init__()
+        W, H, D = width, num_heads, head_dim
+        self.width, self.num_heads, self.head_dim, self.eps = W, H, D, eps
+        f32 = dict(dtype=torch.float32)
+        self.mu = nn.Parameter(torch.zeros(len(self.MIXES), W, **f32), requires_grad=False)
+        self.proj = nn.Parameter(torch.zeros(4, W, H * D), requires_grad=False)
+        self.decay_down = nn.Parameter(torch.zeros(1, W), requires_grad=False)          # [rank, W]
+        self.decay_up = nn.Parameter(torch.zeros(H * D, 1), requires_grad=False)        # [H*D, rank]
+        self.decay_bias = nn.Parameter(torch.zeros(H * D, **f32), requires_grad=False)
+        self.bonus = nn.Parameter(torch.zeros(H, D, **f32), requires_grad=False)
+        self.norm_weight = nn.Parameter(torch.ones(H * D, **f32), requires_grad=False)
+        spec = [("state", (H, D, D)), ("shift", (1, W))]
+        self.slots: List[StateSlots] = [StateSlots(spec) for _ in range(passes)]
+
+    def forward(self, h: torch.Tensor, which: int = 0) -> torch.Tensor:
+        """h [T, W] -> [T, H*D] (input of the output projection); ``which``: the pass whose state
+        is read and advanced."""
+        ctx = get_context()
+        st = self.slots[which]
+        if st.state is None:
+            raise RuntimeError("time mixing needs allocated state slots")
+        T, H, D = h.shape[0], self.num_heads, self.head_dim
+        lay = _layout(ctx)
+        mixes = ops.shift_mix(h, self.mu, st.shift, *lay, row_seq=ctx.row_seq if ctx.is_prefill else None)
+        r, k, v, gate = torch.bmm(mixes[:4], self.proj).unbind(0)
+        low = ops.tanh_cap_(F.linear(mixes[4], self.decay_down), 1.0)
+        o = ops.wkv_scan(r.view(T, H, D), k.view(T, H, D), v.view(T, H, D), F.linear(low, self.decay_up),
+                         self.decay_bias, self.bonus, st.state, *lay)
+        return ops.gated_head_norm(o, self.norm_weight, gate, self.eps, h.dtype, "silu").view(T, H * D)

@@ -124,3 +124,13 @@ def _ensure_builtin() -> None:
         return DanipelForCausalLM
 
     register(["danipel"], danipel_cfg, danipel_class)
+
+    def tedenex_cfg(c, name):
+        from minivllm_amd.models.tedenex import TedenexConfig
+        return TedenexConfig.from_dict(c, name)
+
+    def tedenex_class():
+        from minivllm_amd.models.tedenex import TedenexForCausalLM
+        return TedenexForCausalLM
+
+    register(["tedenex"], tedenex_cfg, tedenex_class)

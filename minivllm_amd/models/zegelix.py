@@ -35,6 +35,7 @@ import torch.nn.functional as F
 
 from minivllm_amd import ops
 from minivllm_amd.layers.attention import SinkAttention
+from minivllm_amd.layers.embedding_head import ScaledTiedHead
 from minivllm_amd.layers.layernorm import GroupRMSNorm
 from minivllm_amd.layers.moe import CappedRoutedExperts
 from minivllm_amd.layers.rglru import RealGatedLRU
@@ -378,48 +379,6 @@ class ZegelixModel(nn.Module):
             if self.layer_hook is not None:
                 self.layer_hook(n, x)
         return x
-
-
-class ScaledTiedHead(nn.Module):
-    """Final RMS norm, then the embedding table itself as the output projection, times a constant.
-    The constant is folded into the norm's fp32 gain (``gain`` = weight * logit_scale), so the
-    logits are rounded once.  Applied to the rows a step wants (each sequence's last row, or the
-    context's ``logit_rows``)."""
-
-    def __init__(self, embedding: nn.Embedding, eps: float, logit_scale: float):
-        super().__init__()
-        self.table = [embedding]                     # not a submodule: the weight is the model's
-        self.eps, self.logit_scale = eps, float(logit_scale)
-        W = embedding.weight.shape[1]
-        self.weight_norm = nn.Parameter(torch.ones(W, dtype=torch.float32), requires_grad=False)
-        self.gain = nn.Parameter(torch.ones(W, dtype=torch.float32), requires_grad=False)
-        self.num_embeddings = embedding.weight.shape[0]
-        self.vocab_start = 0
-
-    @property
-    def weight(self) -> torch.Tensor:
-        return self.table[0].weight
-
-    @torch.no_grad()
-    def load_norm(self, t: torch.Tensor) -> None:
-        self.weight_norm.copy_(t)
-        self.gain.copy_(self.weight_norm * self.logit_scale)
-
-    def select_last(self, hidden: torch.Tensor) -> torch.Tensor:
-        ctx = get_context()
-        if ctx.logit_rows is not None:
-            return hidden.index_select(0, ctx.logit_rows.long())
-        if ctx.is_prefill and ctx.cu_seqlens_q is not None:
-            return hidden.index_select(0, (ctx.cu_seqlens_q[1:] - 1).long())
-        return hidden
-
-    def local_logits(self, hidden: torch.Tensor) -> torch.Tensor:
-        rows = self.select_last(hidden)
-        w = self.weight
-        return F.linear(ops.group_rms_norm(rows, self.gain, 1, self.eps, w.dtype), w)
-
-    def forward(self, hidden: torch.Tensor) -> torch.Tensor:
-        return self.local_logits(hidden)
 
 
 class ZegelixForCausalLM(nn.Module):

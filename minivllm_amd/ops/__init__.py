@@ -253,8 +253,8 @@ def offset_rms_norm(x, w, eps, out_dtype):
     return _seqmix(x).offset_rms_norm(x, w, eps, out_dtype)
 
 
-def post_norm_residual(y, wb, x, eps, w_next, out_dtype):
-    return _seqmix(x).post_norm_residual(y, wb, x, eps, w_next, out_dtype)
+def post_norm_residual(y, wb, x, eps, w_next, out_dtype, plain=False, raw=False, extra=None):
+    return _seqmix(x).post_norm_residual(y, wb, x, eps, w_next, out_dtype, plain, raw, extra)
 
 
 def pair_rope_mix_store(q, k, v, positions, cos_sin, rot_dims, v_first, lam, v_mode,
@@ -266,7 +266,7 @@ def pair_rope_mix_store(q, k, v, positions, cos_sin, rot_dims, v_first, lam, v_m
 def sink_attention_prefill(q, k_cache, v_cache, cu_q, cu_k, block_tables, scale, sink, gate, out,
                            positions=None, max_q=None, row_seq=None, first_seq=0,
                            window=0, keep_first=0, slopes=None, temps=None, softcap=0.0, pool=0,
-                           k_pool=None, v_pool=None):
+                           k_pool=None, v_pool=None, chunk=0):
     """``temps`` [H] fp32: a score multiplier per head; ``softcap`` > 0: score <- softcap
     tanh(score / softcap); ``pool`` > 0 with ``k_pool`` / ``v_pool``: one pooled key / value per
     block of ``pool`` tokens that has passed out of the window as a whole
@@ -276,17 +276,18 @@ def sink_attention_prefill(q, k_cache, v_cache, cu_q, cu_k, block_tables, scale,
     GPU kernels take besides (``hip_hybrid.sink_attention_prefill``); the CPU form derives
     everything from ``cu_q`` / ``cu_k``.  ``sink`` None: no sink term.  ``window`` > 0: a query at
     position i sees key j <= i only if i - j < window or j < keep_first.  ``slopes`` [H] fp32:
-    slope_h * (i - j) is taken off the score."""
+    slope_h * (i - j) is taken off the score.  ``chunk`` > 0: a query sees only keys of its own run of
+    ``chunk`` positions, counted from position 0 of the sequence."""
     if _on_gpu(q):
         return _hybrid().sink_attention_prefill(q, k_cache, v_cache, cu_q, cu_k, block_tables,
                                                 scale, sink, gate, out, positions=positions,
                                                 max_q=max_q, row_seq=row_seq, first_seq=first_seq,
                                                 window=window, keep_first=keep_first, slopes=slopes,
                                                 temps=temps, softcap=softcap, pool=pool,
-                                                k_pool=k_pool, v_pool=v_pool)
+                                                k_pool=k_pool, v_pool=v_pool, chunk=chunk)
     return torch_seqmix.sink_attention_prefill(q, k_cache, v_cache, cu_q, cu_k, block_tables,
                                                scale, sink, gate, out, window, keep_first, slopes,
-                                               temps, softcap, pool, k_pool, v_pool)
+                                               temps, softcap, pool, k_pool, v_pool, chunk)
 
 
 def sink_attention_step(q, k_cache, v_cache, block_tables, row_seq, positions, scale, sink, gate,
@@ -299,7 +300,7 @@ def sink_attention_step(q, k_cache, v_cache, block_tables, row_seq, positions, s
 
 def sink_attention_decode(q, k_cache, v_cache, block_tables, context_lens, scale, sink, gate, out,
                           max_context_len=None, window=0, keep_first=0, slopes=None, temps=None,
-                          softcap=0.0, pool=0, k_pool=None, v_pool=None):
+                          softcap=0.0, pool=0, k_pool=None, v_pool=None, chunk=0):
     """``max_context_len`` (a host integer, an upper bound will do): lets the GPU form size its
     context splits without reading the lengths back."""
     if _on_gpu(q):
@@ -307,10 +308,10 @@ def sink_attention_decode(q, k_cache, v_cache, block_tables, context_lens, scale
                                                scale, sink, gate, out, max_context_len,
                                                window=window, keep_first=keep_first, slopes=slopes,
                                                temps=temps, softcap=softcap, pool=pool,
-                                               k_pool=k_pool, v_pool=v_pool)
+                                               k_pool=k_pool, v_pool=v_pool, chunk=chunk)
     return torch_seqmix.sink_attention_decode(q, k_cache, v_cache, block_tables, context_lens,
                                               scale, sink, gate, out, window, keep_first, slopes,
-                                              temps, softcap, pool, k_pool, v_pool)
+                                              temps, softcap, pool, k_pool, v_pool, chunk)
 
 
 def unit_norm_store(q, k, eps, k_cache, v_cache, slot_mapping):
@@ -485,3 +486,30 @@ def corrected_route(h, router_w, correction, top, identity, scale):
 
 def gelu_tanh_glu(gu, out_dtype):
     return _seqmix(gu).gelu_tanh_glu(gu, out_dtype)
+
+
+# ------------------------------------------------------------------ filtered heads, token shift, wkv
+def conv_norm_store(x, sizes, conv_w, conv_state, qw, kw, eps, k_cache, v_cache, slot_mapping, cu_q,
+                    positions, slots, row_seq=None):
+    """``row_seq`` [T] (GPU, prefill-form steps): the sequence of each row; the CPU form walks
+    ``cu_q``."""
+    a = (x, sizes, conv_w, conv_state, qw, kw, eps, k_cache, v_cache, slot_mapping, cu_q, positions, slots)
+    return _hybrid().conv_norm_store(*a, row_seq) if _on_gpu(x) else torch_seqmix.conv_norm_store(*a)
+
+
+def shift_mix(h, mu, state, cu_q, positions, slots, row_seq=None):
+    """``row_seq``: see ``conv_norm_store``."""
+    a = (h, mu, state, cu_q, positions, slots)
+    return _hybrid().shift_mix(*a, row_seq) if _on_gpu(h) else torch_seqmix.shift_mix(*a)
+
+
+def wkv_scan(r, k, v, w_raw, w_bias, bonus, state, cu_q, positions, slots):
+    return _seqmix(r).wkv_scan(r, k, v, w_raw, w_bias, bonus, state, cu_q, positions, slots)
+
+
+def relu_squared(u, out_dtype):
+    return _seqmix(u).relu_squared(u, out_dtype)
+
+
+def token_gate(z, ids, table, offset, out_dtype):
+    return _seqmix(z).token_gate(z, ids, table, offset, out_dtype)

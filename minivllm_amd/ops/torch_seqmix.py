@@ -45,11 +45,19 @@ def offset_rms_norm(x, w, eps, out_dtype):
     return (xf * torch.rsqrt(xf.pow(2).mean(-1, keepdim=True) + eps) * (1.0 + w.float())).to(out_dtype)
 
 
-def post_norm_residual(y, wb, x, eps, w_next, out_dtype):
-    """``x += norm(y) * (1 + wb)`` in place on the fp32 stream ``x``; with ``w_next`` also returns
-    ``norm(x) * (1 + w_next)`` (the input of the next sublayer)."""
+def post_norm_residual(y, wb, x, eps, w_next, out_dtype, plain=False, raw=False, extra=None):
+    """``x += norm(y) * (1 + wb)`` in place on the fp32 stream ``x`` (``plain``: times wb itself);
+    ``extra`` = (ids [T], table): then ``x += table[ids]``; with ``w_next`` also returns
+    ``norm(x) * (1 + w_next)`` (the input of the next sublayer), with ``raw`` x itself rounded to
+    ``out_dtype``."""
     yf = y.float()
-    x.add_(yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps) * (1.0 + wb.float()))
+    gain = wb.float() if plain else 1.0 + wb.float()
+    x.add_(yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps) * gain)
+    if extra is not None:
+        ids, table = extra
+        x.add_(table[ids.long()].float())
+    if raw:
+        return x.to(out_dtype)
     if w_next is None:
         return None
     return offset_rms_norm(x, w_next, eps, out_dtype)
@@ -112,7 +120,7 @@ def pair_rope_mix_store(q, k, v, positions, cos_sin, rot_dims, v_first, lam, v_m
 
 # ------------------------------------------------------------------ attention with a sink
 def _sink_attend(q, k, v, scale, sink, gate, offset, window=0, keep_first=0, slopes=None,
-                 temps=None, softcap=0.0, pool=0, kp=None, vp=None):
+                 temps=None, softcap=0.0, pool=0, kp=None, vp=None, chunk=0):
     """q [Lq,H,D], k [Lk,G,D], v [Lk,G,E], gate [Lq,H] -> [Lq,H,E] fp32.  Query row i sits at
     position ``offset + i`` and sees key j <= its position; with ``window`` > 0 only keys with
     position - j < window or j < keep_first.  ``slopes`` [H]: slope_h * (position - j) is taken
@@ -120,7 +128,8 @@ def _sink_attend(q, k, v, scale, sink, gate, offset, window=0, keep_first=0, slo
     multiplied by temps[h]; ``softcap`` > 0: score <- softcap tanh(score / softcap), after scale
     and temperature.  ``pool`` > 0 (with a window): ``kp`` [Nb,G,D] / ``vp`` [Nb,G,E] hold one key
     and value per block of ``pool`` tokens; block b joins the softmax of a query at position i
-    when b pool + pool - 1 <= i - window."""
+    when b pool + pool - 1 <= i - window.  ``chunk`` > 0: only keys of the query's own run of
+    ``chunk`` positions (counted from position 0) are seen."""
     Lq, H, _ = q.shape
     Lk, G, _ = k.shape
     r = H // G
@@ -136,6 +145,8 @@ def _sink_attend(q, k, v, scale, sink, gate, offset, window=0, keep_first=0, slo
     hidden = kj > qi
     if window:
         hidden = hidden | ((qi - kj >= window) & (kj >= keep_first))
+    if chunk:
+        hidden = hidden | (torch.div(qi, chunk, rounding_mode="floor") != torch.div(kj, chunk, rounding_mode="floor"))
     hidden = hidden.expand(Lq, Lk)
     if pool and window and kp is not None and kp.shape[0]:
         Nb = kp.shape[0]
@@ -171,7 +182,7 @@ def _pooled(k_pool, v_pool, table, ctx, window, pool):
 
 def sink_attention_prefill(q, k_cache, v_cache, cu_q, cu_k, block_tables, scale, sink, gate, out,
                            window=0, keep_first=0, slopes=None, temps=None, softcap=0.0, pool=0,
-                           k_pool=None, v_pool=None):
+                           k_pool=None, v_pool=None, chunk=0):
     cq, ck = cu_q.tolist(), cu_k.tolist()
     for b in range(len(cq) - 1):
         s, e = cq[b], cq[b + 1]
@@ -183,13 +194,13 @@ def sink_attention_prefill(q, k_cache, v_cache, cu_q, cu_k, block_tables, scale,
         kp, vp = _pooled(k_pool, v_pool, block_tables[b], lk, window, pool)
         out[s:e] = _sink_attend(q[s:e], k, v, scale, sink, None if gate is None else gate[s:e],
                                 lk - (e - s), window, keep_first, slopes, temps, softcap, pool,
-                                kp, vp).to(out.dtype)
+                                kp, vp, chunk).to(out.dtype)
     return out
 
 
 def sink_attention_decode(q, k_cache, v_cache, block_tables, context_lens, scale, sink, gate, out,
                           window=0, keep_first=0, slopes=None, temps=None, softcap=0.0, pool=0,
-                          k_pool=None, v_pool=None):
+                          k_pool=None, v_pool=None, chunk=0):
     for b, L in enumerate(context_lens.tolist()):
         if L <= 0:
             continue
@@ -198,7 +209,7 @@ def sink_attention_decode(q, k_cache, v_cache, block_tables, context_lens, scale
         kp, vp = _pooled(k_pool, v_pool, block_tables[b], L, window, pool)
         out[b:b + 1] = _sink_attend(q[b:b + 1], k, v, scale, sink,
                                     None if gate is None else gate[b:b + 1], L - 1, window,
-                                    keep_first, slopes, temps, softcap, pool, kp, vp).to(out.dtype)
+                                    keep_first, slopes, temps, softcap, pool, kp, vp, chunk).to(out.dtype)
     return out
 
 
@@ -771,3 +782,70 @@ def gelu_tanh_glu(gu, out_dtype):
     """gu [T, 2 C] (gate columns, then up columns; rows may be strided) -> gelu_tanh(gate) * up."""
     C = gu.shape[1] // 2
     return (gelu_tanh(gu[:, :C].float()) * gu[:, C:].float()).to(out_dtype)
+
+
+# ------------------------------------------------------------------ filtered heads, token shift, wkv
+def conv_norm_store(x, sizes, conv_w, conv_state, qw, kw, eps, k_cache, v_cache, slot_mapping, cu_q,
+                    positions, slots):
+    """x [T, >= C]: projected q (H heads of D), k (G of D) and v (G of E) side by side, C = H D + G D +
+    G E, ``sizes`` = (H, G, D, E).  Every channel passes a causal filter over time (``conv_w``
+    [C, taps], no bias; a sequence's last taps-1 inputs live in ``conv_state``, see
+    ``short_conv``); then each q head and k head is divided by its root mean square and multiplied
+    by ``qw`` / ``kw`` [D] (fp32), k and v go to their cache rows (slot < 0: nowhere).  Returns q
+    [T, H, D]."""
+    H, G, D, E = sizes
+    T, C = x.shape[0], H * D + G * D + G * E
+    y = short_conv(x[:, :C], conv_w, None, conv_state, cu_q, positions, slots)
+    q = rms_norm_rows(y[:, :H * D].reshape(T * H, D), qw, eps, x.dtype).view(T, H, D)
+    k = rms_norm_rows(y[:, H * D:(H + G) * D].reshape(T * G, D), kw, eps, torch.float32).view(T, G, D)
+    if k_cache is not None and slot_mapping is not None:
+        _scatter_rows(k_cache, k, slot_mapping)
+        _scatter_rows(v_cache, y[:, (H + G) * D:].view(T, G, E), slot_mapping)
+    return q
+
+
+def shift_mix(h, mu, state, cu_q, positions, slots):
+    """h [T, W], mu [n, W] fp32 -> [n, T, W]: row t of mix i is h_t + (h_(t-1) - h_t) mu[i], with
+    zeros ahead of a sequence's first token.  A sequence's last row lives in ``state``
+    [slots, 1, W] fp32 and is replaced by this step's."""
+    hf = h.float()
+    prev = torch.zeros_like(hf)
+    for s, e, slot, past in _seq_rows(cu_q, positions, slots):
+        if past:
+            prev[s] = state[slot, 0]
+        prev[s + 1:e] = hf[s:e - 1]
+        state[slot, 0] = hf[e - 1]
+    return (hf[None] + (prev - hf)[None] * mu.float()[:, None, :]).to(h.dtype)
+
+
+def wkv_scan(r, k, v, w_raw, w_bias, bonus, state, cu_q, positions, slots):
+    """o = (S + diag(bonus) k v^T)^T r, then S <- diag(w) S + k v^T, with w = exp(-exp(w_raw + w_bias))
+    per head and key channel.  r, k [T,H,D]; v [T,H,E]; w_raw [T,H*D]; bonus [H,D]; ``state``
+    [slots,H,D,E] fp32.  Returns o [T,H,E] fp32."""
+    T, H, D = r.shape
+    E = v.shape[2]
+    rf, kf, vf = r.float(), k.float(), v.float()
+    decay = torch.exp(-torch.exp(w_raw.float().reshape(T, H, D) + w_bias.float().view(H, D)))
+    u = bonus.float().view(H, D, 1)
+    o = torch.zeros(T, H, E, dtype=torch.float32)
+    for s, e, slot, past in _seq_rows(cu_q, positions, slots):
+        S = state[slot].clone() if past else torch.zeros(H, D, E)
+        for t in range(s, e):
+            kv = kf[t][:, :, None] * vf[t][:, None, :]
+            o[t] = torch.einsum("hde,hd->he", S + u * kv, rf[t])
+            S = decay[t][:, :, None] * S + kv
+        state[slot] = S
+    return o
+
+
+# ------------------------------------------------------------------ squared relu, token input of a layer
+def relu_squared(u, out_dtype):
+    """max(u, 0)^2; u may be a strided column block.  Returns a contiguous tensor."""
+    z = torch.clamp(u.float(), min=0.0)
+    return (z * z).to(out_dtype)
+
+
+def token_gate(z, ids, table, offset, out_dtype):
+    """z [T, n] -> gelu_tanh(z) * table[ids, offset:offset + n], element by element."""
+    n = z.shape[1]
+    return (gelu_tanh(z.float()) * table[ids.long(), offset:offset + n].float()).to(out_dtype)
