@@ -17,7 +17,8 @@
 // Options of all three (struct KeyRule): no sink (sink == null: an ordinary softmax; the running
 // maximum then starts at a large negative FINITE number and the sum at 0, so that no path forms
 // inf - inf), a sliding window that keeps the first tokens (a query at position i sees key j <= i
-// only when i - j < window or j < keep_first; keys outside are never loaded), and a distance
+// only when i - j < window or j < keep_first; keys outside are never loaded), chunks (a query sees
+// only keys of its own run of `chunk` positions, counted from position 0), a distance
 // penalty slope_h * (i - j) taken off the score; a multiplier per query head on the scaled score
 // (temps), a tanh soft cap (score <- cap tanh(score / cap), after scale and multiplier), and pooled
 // blocks behind the window: with pool = P > 0 a query at position i also sees ONE key / value row
@@ -41,6 +42,14 @@ struct KeyRule {
     int pool;               // 0: no pooled blocks (needs window > 0 and keep_first == 0)
     int pool_rows;          // pooled rows per page
     long pool_base;         // first pooled row, in rows from the start of the K (and of the V) cache
+    int chunk;              // 0: none (else keep_first == 0 and pool == 0)
+    // the first key a query at position i sees besides kept first tokens and pooled rows; it never
+    // falls as i grows
+    __device__ __forceinline__ int first_key(int i) const {
+        int lo = window > 0 ? max(0, i - window + 1) : 0;
+        if (chunk > 0) lo = max(lo, i / chunk * chunk);
+        return lo;
+    }
     __device__ __forceinline__ float capped(float s) const {
         return softcap > 0.f ? softcap * tanhf(s / softcap) : s;
     }
@@ -61,7 +70,7 @@ struct KeyRule {
 struct VisibleKeys {
     int kept, lo, count;
     __device__ __forceinline__ VisibleKeys(int ctx, const KeyRule& r) {
-        lo = r.window > 0 ? max(0, ctx - r.window) : 0;
+        lo = r.first_key(ctx - 1);
         kept = r.pool > 0 ? r.pooled_for(ctx) : min(r.keep_first, lo);
         count = kept + ctx - lo;
     }
@@ -311,9 +320,10 @@ sink_attention_tiles_kernel(const T* __restrict__ q, long q_row, long q_head,
     const int wg_ctx = start + min(qlen, tile * 128 + 128);            // keys this workgroup needs
     const bool wave_live = tile * 128 + wave * 32 < qlen;
     const int wave_last = start + min(qlen - 1, tile * 128 + wave * 32 + 31);
-    // with a window: the oldest key any query of the workgroup / of the wave still sees
-    const int wg_lo = rule.window > 0 ? max(0, start + tile * 128 - rule.window + 1) : 0;
-    const int wave_lo = rule.window > 0 ? max(0, start + tile * 128 + wave * 32 - rule.window + 1) : 0;
+    // the oldest key any query of the workgroup / of the wave / this lane's query sees (window, chunk)
+    const int wg_lo = rule.first_key(start + tile * 128);
+    const int wave_lo = rule.first_key(start + tile * 128 + wave * 32);
+    const int q_lo = rule.first_key(qpos);
 
     // pooled rows first (those the workgroup's last query takes in), then the tokens
     const int wg_nb = EXT ? rule.pooled_for(wg_ctx) : 0, ptiles = EXT ? (wg_nb + 31) / 32 : 0;
@@ -411,7 +421,7 @@ sink_attention_tiles_kernel(const T* __restrict__ q, long q_row, long q_head,
             for (int r = 0; r < 16; ++r) {
                 const int key = k0 + 8 * (r >> 2) + 4 * half + (r & 3);
                 const bool seen = qok && (pooled ? key < q_nb : (key <= qpos &&
-                                  (rule.window <= 0 || qpos - key < rule.window || key < rule.keep_first)));
+                                  (key >= q_lo || key < rule.keep_first)));
                 const float v = seen ? (EXT ? rule.capped(sacc[r]) : sacc[r]) - (pooled ? 0.f : slope * (float)(qpos - key)) : -INFINITY;
                 sacc[r] = v;
                 mt = fmaxf(mt, v);
@@ -631,6 +641,10 @@ static int launch_split(const void* q, long q_row, long q_head, const void* k_ca
     return HYB_LAUNCH_OK();
 }
 
+static bool chunk_rule_ok(const KeyRule& r) {
+    return r.chunk == 0 || (r.chunk > 0 && r.keep_first == 0 && r.pool == 0);
+}
+
 // pooled blocks need a window, no kept first tokens, no distance penalty, and a place in the caches
 static bool pool_rule_ok(const KeyRule& r) {
     return r.pool == 0 || (r.pool > 0 && r.window > 0 && r.keep_first == 0 && !r.slopes &&
@@ -651,12 +665,12 @@ int hyb_sink_attention_split(const void* q, long q_row, long q_head, const void*
                              const void* gate, long gate_row, void* out, void* ws, float scale,
                              int B, int H, int G, int D, int E, int splits, int window,
                              int keep_first, const void* slopes, int v_stride, const void* temps,
-                             float softcap, int pool, int pool_rows, long pool_base, int dt,
-                             hipStream_t s) {
+                             float softcap, int pool, int pool_rows, long pool_base, int chunk,
+                             int dt, hipStream_t s) {
     const KeyRule rule{window, keep_first, (const float*)slopes, v_stride > 0 ? v_stride : E,
-                       (const float*)temps, softcap, pool, pool_rows, pool_base};
+                       (const float*)temps, softcap, pool, pool_rows, pool_base, chunk};
     if (B <= 0) return 0;
-    if (!pool_rule_ok(rule)) return 1;
+    if (!pool_rule_ok(rule) || !chunk_rule_ok(rule)) return 1;
     if (G <= 0 || H % G || splits < 1 || !hyb_sink_attention_split_ok(D, E)) return 1;
     if (rule.v_stride < E || rule.v_stride % 8) return 1;      // 16-byte runs of a value row
     if (((size_t)k_cache | (size_t)v_cache | (size_t)q) % 16 || (q_row * (dt == 0 ? 2 : 4)) % 16) return 1;
@@ -690,11 +704,11 @@ int hyb_sink_attention_tiles(const void* q, long q_row, long q_head, const void*
                              float scale, int nseq, int seq0, int max_q, int H, int G, int D,
                              int E, int window, int keep_first, const void* slopes, int v_stride,
                              const void* temps, float softcap, int pool, int pool_rows,
-                             long pool_base, int dt, hipStream_t s) {
+                             long pool_base, int chunk, int dt, hipStream_t s) {
     const KeyRule rule{window, keep_first, (const float*)slopes, v_stride > 0 ? v_stride : E,
-                       (const float*)temps, softcap, pool, pool_rows, pool_base};
+                       (const float*)temps, softcap, pool, pool_rows, pool_base, chunk};
     if (nseq <= 0 || max_q <= 0) return 0;
-    if (!pool_rule_ok(rule)) return 1;
+    if (!pool_rule_ok(rule) || !chunk_rule_ok(rule)) return 1;
     if (rule.v_stride < E) return 1;
     if (G <= 0 || H % G || !hyb_sink_attention_tiles_ok(D, E)) return 1;
 #define TILES_ARGS q, q_row, q_head, k_cache, v_cache, block_tables, max_blocks, block_size, cu_q, \
@@ -726,11 +740,11 @@ int hyb_sink_attention_rows(const void* q, long q_row, long q_head, const void* 
                             float scale, long rows, int H, int G, int D, int E, int seq_base,
                             int window, int keep_first, const void* slopes, int v_stride,
                             const void* temps, float softcap, int pool, int pool_rows,
-                            long pool_base, int dt, hipStream_t s) {
+                            long pool_base, int chunk, int dt, hipStream_t s) {
     const KeyRule rule{window, keep_first, (const float*)slopes, v_stride > 0 ? v_stride : E,
-                       (const float*)temps, softcap, pool, pool_rows, pool_base};
+                       (const float*)temps, softcap, pool, pool_rows, pool_base, chunk};
     if (rows <= 0) return 0;
-    if (!pool_rule_ok(rule)) return 1;
+    if (!pool_rule_ok(rule) || !chunk_rule_ok(rule)) return 1;
     if (rule.v_stride < E) return 1;
     if (G <= 0 || H % G || E > NACC * TILE || D > 1024) return 1;
     const int fit = NACC * TILE / E;                     // heads whose output columns fit

@@ -30,28 +30,91 @@ __global__ void offset_rms_norm_kernel(const float* __restrict__ x, const float*
     for (int c = threadIdx.x; c < W; c += blockDim.x) st(out + t * W + c, xr[c] * r * (1.f + w[c]));
 }
 
-// x[t] += y[t] / rms(y[t]) * (1 + wb);  h[t] = x[t] / rms(x[t]) * (1 + wn)   (h optional)
+// x[t] += y[t] / rms(y[t]) * (base + wb) (+ table[ids[t]]);
+// h[t] = x[t] / rms(x[t]) * (1 + wn), or (wn null) x[t] itself               (h, table optional)
+// Any width; the form below keeps the row in registers.
 template <typename T>
 __global__ void post_norm_residual_kernel(const T* __restrict__ y, long y_stride,
-                                          const float* __restrict__ wb, float* __restrict__ x,
-                                          const float* __restrict__ wn, T* __restrict__ h, int W,
-                                          float eps) {
+                                          const float* __restrict__ wb, float base,
+                                          const int* __restrict__ ids, const T* __restrict__ table,
+                                          float* __restrict__ x, const float* __restrict__ wn,
+                                          T* __restrict__ h, int W, float eps) {
     __shared__ float red[16];
     const long t = blockIdx.x;
     const T* yr = y + t * y_stride;
+    const T* er = table ? table + (long)ids[t] * W : nullptr;
     float* xr = x + t * W;
     float s = 0.f;
     for (int c = threadIdx.x; c < W; c += blockDim.x) { const float v = ld(yr + c); s += v * v; }
     const float r = rsqrtf(block_sum(s, red) / (float)W + eps);
     float s2 = 0.f;
     for (int c = threadIdx.x; c < W; c += blockDim.x) {
-        const float v = xr[c] + ld(yr + c) * r * (1.f + wb[c]);
+        float v = xr[c] + ld(yr + c) * r * (base + wb[c]);
+        if (er) v += ld(er + c);
         xr[c] = v;
         s2 += v * v;
+        if (h && !wn) st(h + t * W + c, v);
     }
-    if (!h) return;
+    if (!h || !wn) return;
     const float r2 = rsqrtf(block_sum(s2, red) / (float)W + eps);
     for (int c = threadIdx.x; c < W; c += blockDim.x) st(h + t * W + c, xr[c] * r2 * (1.f + wn[c]));
+}
+
+// The same with NR runs of eight columns per thread (W <= 8 * NR * blockDim.x, whole runs): every
+// load of the row is in flight at once, y and x are read once, x is written once.
+template <typename T, int NR>
+__global__ void __launch_bounds__(256)
+post_norm_residual_runs_kernel(const T* __restrict__ y, long y_stride,
+                               const float* __restrict__ wb, float base,
+                               const int* __restrict__ ids, const T* __restrict__ table,
+                               float* __restrict__ x, const float* __restrict__ wn,
+                               T* __restrict__ h, int W, float eps) {
+    __shared__ float red[16];
+    const long t = blockIdx.x;
+    float yv[NR][8], xv[NR][8], wv[NR][8], ev[NR][8];
+    const T* er = table ? table + (long)ids[t] * W : nullptr;
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+        const int c = (threadIdx.x + i * blockDim.x) * 8;
+        if (c < W) {
+            load_run<T, 8>(y + t * y_stride + c, yv[i]);
+            load_run<float, 8>(x + t * W + c, xv[i]);
+            load_run<float, 8>(wb + c, wv[i]);
+            if (er) load_run<T, 8>(er + c, ev[i]);
+#pragma unroll
+            for (int j = 0; j < 8; ++j) s += yv[i][j] * yv[i][j];
+        }
+    }
+    const float r = rsqrtf(block_sum(s, red) / (float)W + eps);
+    float s2 = 0.f;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+        const int c = (threadIdx.x + i * blockDim.x) * 8;
+        if (c < W) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                float v = xv[i][j] + yv[i][j] * r * (base + wv[i][j]);
+                if (er) v += ev[i][j];
+                xv[i][j] = v;
+                s2 += v * v;
+            }
+            store_run8<float>(x + t * W + c, xv[i]);
+            if (h && !wn) store_run8<T>(h + t * W + c, xv[i]);
+            if (h && wn) load_run<float, 8>(wn + c, wv[i]);
+        }
+    }
+    if (!h || !wn) return;
+    const float r2 = rsqrtf(block_sum(s2, red) / (float)W + eps);
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+        const int c = (threadIdx.x + i * blockDim.x) * 8;
+        if (c < W) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) xv[i][j] *= r2 * (1.f + wv[i][j]);
+            store_run8<T>(h + t * W + c, xv[i]);
+        }
+    }
 }
 
 // Per token: rotate q in place (pairs (2i, 2i+1) of the first rot entries of each head), rotate k
@@ -257,12 +320,29 @@ int hyb_offset_rms_norm(const void* x, const void* w, void* out, long T_, int W,
     return HYB_LAUNCH_OK();
 }
 
-int hyb_post_norm_residual(const void* y, long y_stride, const void* wb, void* x, const void* wn,
-                           void* h, long T_, int W, float eps, int dt, hipStream_t s) {
+// base: 1 (wb is an offset from one) or 0 (wb is the gain); table (with ids [T]): rows added to the
+// stream besides; h with wn null: the stream itself, narrowed.
+int hyb_post_norm_residual(const void* y, long y_stride, const void* wb, float base, const void* ids,
+                           const void* table, void* x, const void* wn, void* h, long T_, int W,
+                           float eps, int dt, hipStream_t s) {
     if (T_ <= 0) return 0;
+    if (table && !ids) return 1;
+    const size_t align = (size_t)y | (size_t)wb | (size_t)table | (size_t)x | (size_t)wn | (size_t)h;
+#define PNR_ARGS (const T*)y, y_stride, (const float*)wb, base, (const int*)ids, (const T*)table, \
+                 (float*)x, (const float*)wn, (T*)h, W, eps
+#define PNR_RUNS(NR)                                                                               \
+    HYB_DISPATCH(dt, hipLaunchKernelGGL((post_norm_residual_runs_kernel<T, NR>), dim3(T_),         \
+                                        dim3(((W / 8 + NR - 1) / NR + 63) / 64 * 64), 0, s, PNR_ARGS))
+    if (W % 8 == 0 && W <= 8192 && y_stride % 8 == 0 && align % 16 == 0) {
+        if (W <= 2048) PNR_RUNS(1);
+        else if (W <= 4096) PNR_RUNS(2);
+        else PNR_RUNS(4);
+        return HYB_LAUNCH_OK();
+    }
     HYB_DISPATCH(dt, hipLaunchKernelGGL(post_norm_residual_kernel<T>, dim3(T_),
-                                        dim3(threads_for(W)), 0, s, (const T*)y, y_stride,
-                                        (const float*)wb, (float*)x, (const float*)wn, (T*)h, W, eps));
+                                        dim3(threads_for(W)), 0, s, PNR_ARGS));
+#undef PNR_RUNS
+#undef PNR_ARGS
     return HYB_LAUNCH_OK();
 }
 

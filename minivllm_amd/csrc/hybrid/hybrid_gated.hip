@@ -9,7 +9,7 @@
 //   chosen_route            router logits + bias, top logits, softmax over the chosen, gate rows
 //   capped_glu_route_scale  w * min(g, L) sigmoid(slope min(g, L)) (clamp(u, -L, L) + 1)
 // Angles, gates, decays, state, router and every transcendental in fp32.
-#include "hybrid_common.h"
+#include "hybrid_conv.h"
 
 using namespace hyb;
 
@@ -272,39 +272,6 @@ __global__ void short_conv_kernel(const T* __restrict__ x, long x_stride, const 
     }
 }
 
-// The kept inputs after the step: grid (channel chunks, sequences); runs after every row has read.
-template <typename T>
-__global__ void short_conv_tail_kernel(const T* __restrict__ x, long x_stride, float* __restrict__ tail,
-                                       const int* __restrict__ cu_q, const int* __restrict__ positions,
-                                       const int* __restrict__ slots, int C, int taps) {
-    const int b = blockIdx.y;
-    const int c = blockIdx.x * blockDim.x + threadIdx.x;
-    if (c >= C) return;
-    const int slot = slots[b];
-    if (slot < 0) return;
-    const long s0 = cu_q ? cu_q[b] : b, e0 = cu_q ? cu_q[b + 1] : b + 1;
-    const int n = (int)(e0 - s0);
-    if (n <= 0) return;
-    const int p0 = positions[s0], keep = taps - 1;
-    float* tl = tail + (long)slot * keep * C + c;
-    for (int i = 0; i < keep; ++i) {                  // ascending: reads never trail the writes
-        const int off = n - keep + i;                 // row offset inside the step
-        float v;
-        if (off >= 0) v = ld(x + (s0 + off) * x_stride + c);
-        else v = (p0 + off >= 0) ? tl[(long)(i + n) * C] : 0.f;
-        tl[(long)i * C] = v;
-    }
-}
-
-// sigmoid on the hardware exponential and reciprocal (both within a few ulp): the scan evaluates
-// three per element and pass
-__device__ __forceinline__ float fast_sigmoid(float z) { return __fdividef(1.f, 1.f + __expf(-z)); }
-
-// 0.5 z (1 + tanh(a)) = z sigmoid(2 a), a = sqrt(2/pi) (z + 0.044715 z^3)
-__device__ __forceinline__ float gelu_tanh_(float z) {
-    return z * fast_sigmoid(1.5957691216057308f * (z + 0.044715f * z * z * z));
-}
-
 // 1 - exp(t) for t <= 0 without cancellation: the series next to zero, 1 - exp(t) elsewhere
 __device__ __forceinline__ float one_minus_exp(float t, float e) {
     const float series = -t * (1.f + t * (0.5f + t * (1.f / 6.f + t * (1.f / 24.f + t * (1.f / 120.f +
@@ -547,7 +514,7 @@ int hyb_short_conv(const void* x, long x_stride, const void* w, const void* bias
     if (taps > 1 && B > 0)
         HYB_DISPATCH(dt, hipLaunchKernelGGL(short_conv_tail_kernel<T>, dim3(bx, B), dim3(th), 0, s,
                                             (const T*)x, x_stride, (float*)tail, (const int*)cu_q,
-                                            (const int*)positions, (const int*)slots, C, taps));
+                                            (const int*)positions, (const int*)slots, C, taps, 0));
     return HYB_LAUNCH_OK();
 }
 

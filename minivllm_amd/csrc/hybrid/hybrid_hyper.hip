@@ -221,9 +221,6 @@ corrected_route_kernel(const T* __restrict__ h, const float* __restrict__ wr,
     if (lane == 0) row[NE] = ident;
 }
 
-__device__ __forceinline__ float gelu_tanh_(float z) {
-    return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-}
 
 // gu row = [gate C | up C]; act dense [T, C]; VEC columns per thread (8: aligned 16-byte runs)
 template <typename T, int VEC>

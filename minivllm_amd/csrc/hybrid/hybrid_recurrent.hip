@@ -1,10 +1,11 @@
 // Gated outer-product recurrences with a fp32 matrix state S [D, E] per (sequence, head), for
-// prefill portions and single decode tokens alike.  One kernel template, three rules:
+// prefill portions and single decode tokens alike.  One kernel template, four rules:
 //
 //   GLA     S <- diag(alpha) S + k v^T;  o = S^T q          alpha = sigmoid(z + b)^(1/tau) per key channel
 //   CDELTA  S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q     g per key channel
 //   MLSTM   m' = max(f + m, i);  S <- e^(f+m-m') S + e^(i-m') k v^T;  n likewise with k alone;
 //           o = S^T q / (max(|n . q|, e^(-m')) + 1e-6)       i, f soft-capped log gates
+//   WKV     o = (S + diag(u) k v^T)^T q;  S <- diag(w) S + k v^T         w = exp(-exp(z + b)) per key channel
 //
 // A state column S[:, e] evolves independently of the others, so a column is owned by LPC
 // neighbouring lanes (4, 8 or 16), lane r holding d in [r*NR, (r+1)*NR) in registers
@@ -15,7 +16,7 @@
 // has few (sequence, head) pairs (prompt portions).  The tokens' operands are staged through LDS
 // in chunks of CT tokens, double-buffered: k, q (and the decay vector) of the head as padded
 // [token][group lane] slices read with 16-byte LDS loads, v of the workgroup's columns, and the
-// per-token scalars.  GLA and
+// per-token scalars.  GLA, WKV and
 // MLSTM read the raw projections (bfloat16 or float rows of a wider projection output) and do
 // the gates' fp32 arithmetic while staging; CDELTA reads the fp32 outputs of delta_prepare.
 // MLSTM's running maximum is a sequential max-plus chain over tokens: wave 0 walks it once per
@@ -30,14 +31,15 @@
 
 using namespace hyb;
 
-enum ScanRule { GLA = 0, CDELTA = 1, MLSTM = 2 };
+enum ScanRule { GLA = 0, CDELTA = 1, MLSTM = 2, WKV = 3 };
 
 struct ScanArgs {
     const void *q, *k, *v;          // rows of [*, D] / [*, E] heads; element strides per token below
     long q_row, k_row, v_row;
-    const void* a;                  // GLA: raw decay pre-activation [T, H*D]; CDELTA: decay fp32 [T, H*D]
+    const void* a;                  // GLA, WKV: raw decay pre-activation [T, H*D]; CDELTA: decay fp32 [T, H*D]
     long a_row;
-    const float* a_bias;            // GLA [H*D]
+    const float* a_bias;            // GLA, WKV [H*D]
+    const float* bonus;             // WKV [H*D]: the weight of the current token's k v^T in its own output
     float tau_inv;
     const void *gi, *gf;            // MLSTM: raw gate pre-activations [T, H]
     long g_row;
@@ -50,6 +52,8 @@ struct ScanArgs {
     int H, G, D, E;
     float qscale;
 };
+
+__device__ __forceinline__ float wkv_decay_(float z) { return expf(-expf(z)); }
 
 __device__ __forceinline__ float logsigmoidf_(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
 
@@ -102,6 +106,12 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
     const TI* kp = (const TI*)a.k;
     const TI* vp = (const TI*)a.v;
 
+    float U[MODE == WKV ? NR : 1];
+    if constexpr (MODE == WKV) {
+#pragma unroll
+        for (int i = 0; i < NR; ++i) U[i] = d0 + i < D ? a.bonus[h * D + d0 + i] : 0.f;
+    }
+
     if (n == 1) {
         // A single token (decode rows, one-token portions): k, q and the decay vector of the head
         // (and MLSTM's three factors) are worked out once per workgroup into LDS, every lane then
@@ -117,6 +127,8 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
                 else if constexpr (MODE == GLA)
                     v = expf(logsigmoidf_(ld((const TI*)a.a + t * a.a_row + (long)h * D + d) +
                                           a.a_bias[h * D + d]) * a.tau_inv);
+                else if constexpr (MODE == WKV)
+                    v = wkv_decay_(ld((const TI*)a.a + t * a.a_row + (long)h * D + d) + a.a_bias[h * D + d]);
                 else if constexpr (MODE == CDELTA) v = ((const float*)a.a)[t * a.a_row + (long)h * D + d];
             }
             sm[i] = v;
@@ -174,6 +186,13 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
                 S[i] += kk[i] * u;
                 po += S[i] * qq[i];
             }
+        } else if constexpr (MODE == WKV) {
+#pragma unroll
+            for (int i = 0; i < NR; ++i) {
+                const float kv = kk[i] * ve;
+                po += (S[i] + U[i] * kv) * qq[i];
+                S[i] = gg[i] * S[i] + kv;
+            }
         } else {
 #pragma unroll
             for (int i = 0; i < NR; ++i) {
@@ -218,7 +237,7 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
     constexpr bool HAS_AUX = MODE != CDELTA;
     int goff[NLD];                  // element offset from the chunk's first row (< 0: the item is 0)
     int ldso[NLD];                  // where it goes in the LDS buffer (< 0: nowhere)
-    float aux[HAS_AUX ? NLD : 1];   // GLA: the decay channel's bias; MLSTM: the gate's bias
+    float aux[HAS_AUX ? NLD : 1];   // GLA, WKV: the decay channel's bias; MLSTM: the gate's bias
     auto item_tok = [&](int x) {    // token-in-chunk of item x (shifts: every size is a power of two)
         const int j = tid + x * 256;
         if (x < X_IMG) return (j % IMG_ITEMS) / (LPC * NR);
@@ -238,7 +257,7 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
                 else if (which == 1) goff[x] = tok * (int)a.q_row + g * D + d;
                 else {
                     goff[x] = tok * (int)a.a_row + h * D + d;
-                    if constexpr (MODE == GLA) aux[x] = a.a_bias[h * D + d];
+                    if constexpr (MODE == GLA || MODE == WKV) aux[x] = a.a_bias[h * D + d];
                 }
             }
         } else if (x < X_IMG + X_V) {
@@ -294,6 +313,8 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
                     if (which == 1) v *= a.qscale;
                     if constexpr (MODE == GLA)
                         if (which == 2) v = expf(logsigmoidf_(v + aux[x]) * a.tau_inv);
+                    if constexpr (MODE == WKV)
+                        if (which == 2) v = wkv_decay_(v + aux[x]);
                 } else if (x >= X_IMG + X_V) {
                     if constexpr (MODE == MLSTM) {
                         v = a.cap * tanhf((v + aux[x]) / a.cap);
@@ -398,6 +419,13 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
                         for (int i = 0; i < NR; ++i) {
                             S[i] += kk[i] * u;
                             o4[i & 3] += S[i] * qq[i];
+                        }
+                    } else if constexpr (MODE == WKV) {
+#pragma unroll
+                        for (int i = 0; i < NR; ++i) {
+                            const float kv = kk[i] * ve;
+                            o4[i & 3] += (S[i] + U[i] * kv) * qq[i];
+                            S[i] = gg[i] * S[i] + kv;
                         }
                     } else {
 #pragma unroll
@@ -510,6 +538,21 @@ int hyb_gla_scan(const void* q, const void* k, const void* v, long q_row, long k
     a.slots = (const int*)slots; a.o = (float*)o; a.H = H; a.G = H; a.D = D; a.E = E;
     a.qscale = 1.f / sqrtf((float)D);
     HYB_DISPATCH(dt, return (scan_by_size<T, GLA>(a, B, s)));
+    return 1;
+}
+
+// As hyb_gla_scan with the rule WKV: w_bias, bonus [H*D]; r and k are taken as they are (no D^-1/2).
+int hyb_wkv_scan(const void* r, const void* k, const void* v, long r_row, long k_row, long v_row,
+                 const void* w_raw, long w_row, const void* w_bias, const void* bonus, void* state,
+                 const void* cu_q, const void* positions, const void* slots, void* o, int B, int H,
+                 int D, int E, int dt, hipStream_t s) {
+    ScanArgs a{};
+    a.q = r; a.k = k; a.v = v; a.q_row = r_row; a.k_row = k_row; a.v_row = v_row;
+    a.a = w_raw; a.a_row = w_row; a.a_bias = (const float*)w_bias; a.bonus = (const float*)bonus;
+    a.state = (float*)state; a.cu_q = (const int*)cu_q; a.positions = (const int*)positions;
+    a.slots = (const int*)slots; a.o = (float*)o; a.H = H; a.G = H; a.D = D; a.E = E;
+    a.qscale = 1.f;
+    HYB_DISPATCH(dt, return (scan_by_size<T, WKV>(a, B, s)));
     return 1;
 }
 

@@ -308,7 +308,7 @@ class FilteredHeads(nn.Module):
         self.conv_weight = nn.Parameter(torch.zeros(self.channels, self.taps, **f32), requires_grad=False)
         self.q_norm = nn.Parameter(torch.ones(D, **f32), requires_grad=False)
         self.k_norm = nn.Parameter(torch.ones(D, **f32), requires_grad=False)
-        spec = [("conv_state", (self.taps - 1, self.channels))] if self.taps > 1 else []
+        spec = [("conv_state", (self.taps - 1, self.channels))]       # (empty rows for a single tap)
         self.slots = [StateSlots(spec) for _ in range(passes)]
 
     def forward(self, proj: torch.Tensor, core: SinkAttention, which: int = 0) -> torch.Tensor:
@@ -317,8 +317,8 @@ class FilteredHeads(nn.Module):
         ctx = get_context()
         pre = ctx.is_prefill
         return ops.conv_norm_store(proj, self.sizes, self.conv_weight,
-                                   self.slots[which].conv_state if self.taps > 1 else None, self.q_norm,
-                                   self.k_norm, self.eps, core.k_cache, core.v_cache, ctx.slot_mapping,
+                                   self.slots[which].conv_state, self.q_norm, self.k_norm, self.eps,
+                                   core.k_cache, core.v_cache, ctx.slot_mapping,
                                    ctx.cu_seqlens_q if pre else None, ctx.positions, ctx.state_slots,
                                    row_seq=ctx.row_seq if pre else None)
 

@@ -181,7 +181,7 @@ class TedenexAttentionMixer(nn.Module):
         return list(self.cores)
 
     def state_cores(self):
-        return list(self.heads.slots) if self.heads.taps > 1 else []
+        return list(self.heads.slots)
 
     def forward(self, h: torch.Tensor, which: int) -> torch.Tensor:
         core = self.cores[which]

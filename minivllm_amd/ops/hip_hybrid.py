@@ -32,13 +32,14 @@ def _sig(name, *argtypes):
 
 _embed = _sig("hyb_embed_sum", _P, _P, _P, _P, _P, _L, _I, _F, _I, _P)
 _norm = _sig("hyb_offset_rms_norm", _P, _P, _P, _L, _I, _F, _I, _P)
-_post = _sig("hyb_post_norm_residual", _P, _L, _P, _P, _P, _P, _L, _I, _F, _I, _P)
+_post = _sig("hyb_post_norm_residual", _P, _L, _P, _F, _P, _P, _P, _P, _P, _L, _I, _F, _I, _P)
 _rope = _sig("hyb_pair_rope_mix_store", _P, _P, _P, _L, _P, _P, _I, _P, _P, _I, _P, _P, _P, _L,
              _I, _I, _I, _I, _I, _P)
 _ghn = _sig("hyb_gated_head_norm", _P, _P, _P, _L, _P, _L, _I, _I, _F, _I, _I, _I, _P)
 _route = _sig("hyb_grouped_route", _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _I, _P)
 _gelu = _sig("hyb_gelu_route_scale", _P, _P, _P, _L, _I, _I, _I, _P)
-_POOL = (_P, _F, _I, _I, _L)        # head temperatures, soft cap, pool, pooled rows per page, first pooled row
+# head temperatures, soft cap, pool, pooled rows per page, first pooled row, chunk
+_POOL = (_P, _F, _I, _I, _L, _I)
 _attn = _sig("hyb_sink_attention_rows", _P, _L, _L, _P, _P, _P, _I, _I, _P, _P, _I, _P, _P, _L, _P,
              _F, _L, _I, _I, _I, _I, _I, _I, _I, _P, _I, *_POOL, _I, _P)
 _tiles = _sig("hyb_sink_attention_tiles", _P, _L, _L, _P, _P, _P, _I, _I, _P, _P, _P, _P, _L, _P, _F,
@@ -85,6 +86,12 @@ _hyp = _sig("hyb_hyper_update_norm", _P, _L, _L, _P, _P, _L, _P, _L, _P, _L, _P,
 _cor = _sig("hyb_corrected_route", _P, _P, _P, _P, _L, _I, _I, _I, _I, _F, _I, _P)
 _gtg = _sig("hyb_gelu_tanh_glu", _P, _L, _P, _L, _I, _I, _P)
 
+_cns = _sig("hyb_conv_norm_store", _P, _L, _P, _P, _P, _P, _F, _P, _P, _P, _P, _P, _P, _P, _P, _L, _I, _I, _I,
+            _I, _I, _I, _I, _P)
+_smx = _sig("hyb_shift_mix", _P, _P, _P, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _P)
+_rsq = _sig("hyb_relu_squared", _P, _L, _P, _L, _I, _I, _P)
+_tgt = _sig("hyb_token_gate", _P, _L, _P, _P, _L, _L, _P, _L, _I, _I, _P)
+_wkv = _sig("hyb_wkv_scan", _P, _P, _P, _L, _L, _L, _P, _L, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P)
 _lat = _sig("hyb_latent_attention", _P, _L, _L, _P, _L, _L, _P, _P, _I, _I, _P, _P, _P, _P, _P, _L, _L, _P,
             _F, _I, _I, _I, _I, _I, _I, _I, _P)
 _lat_ok = _lib.hyb_latent_attention_ok
@@ -152,13 +159,18 @@ def offset_rms_norm(x, w, eps, out_dtype):
     return out
 
 
-def post_norm_residual(y, wb, x, eps, w_next, out_dtype):
+def post_norm_residual(y, wb, x, eps, w_next, out_dtype, plain=False, raw=False, extra=None):
     x = _f32(x)
     T, W = x.shape
-    assert y.shape == x.shape and y.stride(-1) == 1 and y.dtype == out_dtype
-    h = torch.empty((T, W), dtype=out_dtype, device=x.device) if w_next is not None else None
-    _check(_post(y.data_ptr(), y.stride(0), _f32(wb).data_ptr(), x.data_ptr(),
-                 _ptr(w_next), _ptr(h), T, W, eps, _dt(y), _stream()), "post_norm_residual")
+    assert y.shape == x.shape and y.stride(-1) == 1 and y.dtype == out_dtype and wb.numel() == W
+    assert not (raw and w_next is not None)
+    h = torch.empty((T, W), dtype=out_dtype, device=x.device) if raw or w_next is not None else None
+    ids, table = extra if extra is not None else (None, None)
+    if table is not None:
+        assert table.is_contiguous() and table.shape[1] == W and table.dtype == y.dtype and ids.shape[0] >= T
+    _check(_post(y.data_ptr(), _rows(y), _f32(wb).data_ptr(), 0.0 if plain else 1.0, _ptr(_i32(ids)),
+                 _ptr(table), x.data_ptr(), _ptr(w_next), _ptr(h), T, W, eps, _dt(y), _stream()),
+           "post_norm_residual")
     return h
 
 
@@ -228,7 +240,7 @@ def _pool_args(k_cache, v_cache, vs, H, temps, softcap, pool, k_pool, v_pool):
 
 def _attention_rows(q, k_cache, v_cache, block_tables, row_seq, lens, len_add, scale, sink, gate, out,
                     seq_base=0, window=0, keep_first=0, slopes=None, temps=None, softcap=0.0, pool=0,
-                    k_pool=None, v_pool=None):
+                    k_pool=None, v_pool=None, chunk=0):
     T, H, D = q.shape
     G, E = k_cache.shape[2], v_cache.shape[3]
     assert q.stride(2) == 1 and out.is_contiguous() and out.shape == (T, H, E) and out.dtype == q.dtype
@@ -243,7 +255,7 @@ def _attention_rows(q, k_cache, v_cache, block_tables, row_seq, lens, len_add, s
                  _f32(sink).data_ptr() if sink is not None else None,
                  _ptr(gate), gate.stride(0) if gate is not None else 0, out.data_ptr(), scale, T,
                  H, G, D, E, seq_base, int(window), int(keep_first), _slopes(slopes, H), vs,
-                 *_pool_args(k_cache, v_cache, vs, H, temps, softcap, pool, k_pool, v_pool), _dt(q),
+                 *_pool_args(k_cache, v_cache, vs, H, temps, softcap, pool, k_pool, v_pool), int(chunk), _dt(q),
                  _stream()), "sink_attention")
     return out
 
@@ -260,7 +272,7 @@ def sink_attention_step(q, k_cache, v_cache, block_tables, row_seq, positions, s
 def sink_attention_prefill(q, k_cache, v_cache, cu_q, cu_k, block_tables, scale, sink, gate, out,
                            positions=None, max_q=None, row_seq=None, first_seq=0,
                            window=0, keep_first=0, slopes=None, temps=None, softcap=0.0, pool=0,
-                           k_pool=None, v_pool=None):
+                           k_pool=None, v_pool=None, chunk=0):
     """The prompt portions of a step: sequence b owns rows cu_q[b] .. cu_q[b+1] (absolute rows
     of q / out / positions) and block table row b.  Runs the matrix-core tile kernel (fp32
     scores, weights and sums); head sizes it has no instance for go row by row.  ``cu_k`` is
@@ -275,7 +287,7 @@ def sink_attention_prefill(q, k_cache, v_cache, cu_q, cu_k, block_tables, scale,
         return sink_attention_step(q, k_cache, v_cache, block_tables, row_seq, positions, scale,
                                    sink, gate, out, seq_base=first_seq, window=window,
                                    keep_first=keep_first, slopes=slopes, temps=temps,
-                                   softcap=softcap, pool=pool, k_pool=k_pool, v_pool=v_pool)
+                                   softcap=softcap, pool=pool, k_pool=k_pool, v_pool=v_pool, chunk=chunk)
     if max_q is None:
         max_q = int((cu_q[1:] - cu_q[:-1]).max())
     assert q.stride(2) == 1 and out.is_contiguous() and out.shape == (T, H, E) and out.dtype == q.dtype
@@ -290,7 +302,7 @@ def sink_attention_prefill(q, k_cache, v_cache, cu_q, cu_k, block_tables, scale,
                   _f32(sink).data_ptr() if sink is not None else None,
                   _ptr(gate), gate.stride(0) if gate is not None else 0, out.data_ptr(), scale,
                   nseq, 0, max_q, H, G, D, E, int(window), int(keep_first), _slopes(slopes, H), vs,
-                  *_pool_args(k_cache, v_cache, vs, H, temps, softcap, pool, k_pool, v_pool),
+                  *_pool_args(k_cache, v_cache, vs, H, temps, softcap, pool, k_pool, v_pool), int(chunk),
                   _dt(q), _stream()), "sink_attention_prefill")
     return out
 
@@ -311,7 +323,7 @@ def decode_splits(batch: int, kv_heads: int, heads: int, max_context_len) -> int
 
 def sink_attention_decode(q, k_cache, v_cache, block_tables, context_lens, scale, sink, gate, out,
                           max_context_len=None, window=0, keep_first=0, slopes=None, temps=None,
-                          softcap=0.0, pool=0, k_pool=None, v_pool=None):
+                          softcap=0.0, pool=0, k_pool=None, v_pool=None, chunk=0):
     """Single next tokens: row b is sequence b with ``context_lens[b]`` keys.  Head sizes the
     split-context kernel has an instance for (D in 64 / 128 / 256, E in 64 / 128) stream K / V
     rows with coalesced 16-byte loads over several workgroups per sequence and are merged by a
@@ -326,6 +338,8 @@ def sink_attention_decode(q, k_cache, v_cache, block_tables, context_lens, scale
         seen = max_context_len
         if window and seen:           # what a row can see bounds the useful splits
             seen = min(int(seen), int(window) + int(keep_first) + (int(seen) // pool if pool else 0))
+        if chunk and seen:
+            seen = min(int(seen), int(chunk))
         splits = decode_splits(B, G, H, seen)
         ws = torch.empty((B * H * splits * (E + 2),), dtype=torch.float32, device=q.device)
         if gate is not None:
@@ -337,12 +351,13 @@ def sink_attention_decode(q, k_cache, v_cache, block_tables, context_lens, scale
                       _ptr(gate), gate.stride(0) if gate is not None else 0, out.data_ptr(),
                       ws.data_ptr(), scale, B, H, G, D, E, splits, int(window), int(keep_first),
                       _slopes(slopes, H), vs,
-                      *_pool_args(k_cache, v_cache, vs, H, temps, softcap, pool, k_pool, v_pool),
+                      *_pool_args(k_cache, v_cache, vs, H, temps, softcap, pool, k_pool, v_pool), int(chunk),
                       _dt(q), _stream()),
                "sink_attention_decode")
         return out
     return _attention_rows(q, k_cache, v_cache, block_tables, None, context_lens, 0, scale, sink,
-                           gate, out, 0, window, keep_first, slopes, temps, softcap, pool, k_pool, v_pool)
+                           gate, out, 0, window, keep_first, slopes, temps, softcap, pool, k_pool, v_pool,
+                           chunk)
 
 
 # ------------------------------------------------------------------ gated delta rule
@@ -884,3 +899,74 @@ def gelu_tanh_glu(gu, out_dtype):
     act = torch.empty((T, C), dtype=out_dtype, device=gu.device)
     _check(_gtg(gu.data_ptr(), _rows(gu), act.data_ptr(), T, C, _dt(gu), _stream()), "gelu_tanh_glu")
     return act
+
+
+# ------------------------------------------------------------------ filtered heads, token shift, wkv
+def conv_norm_store(x, sizes, conv_w, conv_state, qw, kw, eps, k_cache, v_cache, slot_mapping, cu_q,
+                    positions, slots, row_seq=None):
+    H, G, D, E = sizes
+    T, C = x.shape[0], (H + G) * D + G * E
+    taps = _f32(conv_w).shape[1]
+    assert x.stride(1) == 1 and x.shape[1] >= C and conv_w.shape[0] == C and qw.numel() == D and kw.numel() == D
+    if cu_q is not None:
+        assert row_seq is not None and row_seq.shape[0] >= T, "prefill-form steps pass the sequence of each row"
+    if taps > 1:
+        assert _f32(conv_state).shape[1:] == (taps - 1, C)
+    if k_cache is not None:
+        assert k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dtype == x.dtype \
+            and v_cache.dtype == x.dtype and k_cache.shape[2:] == (G, D) and v_cache.shape[2:] == (G, E)
+    assert positions.shape[0] >= T and (slot_mapping is None or slot_mapping.shape[0] >= T)
+    q = torch.empty((T, H, D), dtype=x.dtype, device=x.device)
+    _check(_cns(x.data_ptr(), _rows(x), conv_w.data_ptr(), _ptr(conv_state) if taps > 1 else None,
+                _f32(qw).data_ptr(), _f32(kw).data_ptr(), eps, q.data_ptr(), _ptr(k_cache), _ptr(v_cache),
+                _ptr(_i32(slot_mapping)), _ptr(_i32(cu_q)), _i32(positions).data_ptr(),
+                _i32(slots).data_ptr(), _ptr(_i32(row_seq)) if cu_q is not None else None, T,
+                slots.shape[0], H, G, D, E, taps, _dt(x), _stream()), "conv_norm_store")
+    return q
+
+
+def shift_mix(h, mu, state, cu_q, positions, slots, row_seq=None):
+    T, W = h.shape
+    n = _f32(mu).shape[0]
+    assert h.is_contiguous() and mu.shape[1] == W and _f32(state).shape[1:] == (1, W) and positions.shape[0] >= T
+    if cu_q is not None:
+        assert row_seq is not None and row_seq.shape[0] >= T, "prefill-form steps pass the sequence of each row"
+    out = torch.empty((n, T, W), dtype=h.dtype, device=h.device)
+    _check(_smx(h.data_ptr(), mu.data_ptr(), state.data_ptr(), _ptr(_i32(cu_q)), _i32(positions).data_ptr(),
+                _i32(slots).data_ptr(), _ptr(_i32(row_seq)) if cu_q is not None else None, out.data_ptr(), T,
+                slots.shape[0], W, n, _dt(h), _stream()), "shift_mix")
+    return out
+
+
+def wkv_scan(r, k, v, w_raw, w_bias, bonus, state, cu_q, positions, slots):
+    T, H, D = r.shape
+    E = v.shape[2]
+    assert state.shape[1:] == (H, D, E) and w_raw.shape == (T, H * D) and w_raw.stride(1) == 1
+    assert k.dtype == r.dtype and v.dtype == r.dtype and w_raw.dtype == r.dtype
+    assert w_bias.numel() == H * D and bonus.numel() == H * D
+    o = torch.zeros((T, H, E), dtype=torch.float32, device=r.device)
+    _check(_wkv(r.data_ptr(), k.data_ptr(), v.data_ptr(), _heads_view(r, D), _heads_view(k, D),
+                _heads_view(v, E), w_raw.data_ptr(), _rows(w_raw), _f32(w_bias).data_ptr(),
+                _f32(bonus).data_ptr(), _f32(state).data_ptr(), _ptr(_i32(cu_q)),
+                _i32(positions).data_ptr(), _i32(slots).data_ptr(), o.data_ptr(), slots.shape[0], H, D, E,
+                _dt(r), _stream()), "wkv_scan")
+    return o
+
+
+# ------------------------------------------------------------------ squared relu, token input of a layer
+def relu_squared(u, out_dtype):
+    T, n = u.shape
+    assert u.stride(1) == 1 and u.dtype == out_dtype
+    act = torch.empty((T, n), dtype=out_dtype, device=u.device)
+    _check(_rsq(u.data_ptr(), _rows(u), act.data_ptr(), T, n, _dt(u), _stream()), "relu_squared")
+    return act
+
+
+def token_gate(z, ids, table, offset, out_dtype):
+    T, n = z.shape
+    assert z.stride(1) == 1 and z.dtype == out_dtype and table.dtype == out_dtype and table.stride(1) == 1
+    assert ids.shape[0] >= T and 0 <= offset and offset + n <= table.shape[1]
+    out = torch.empty((T, n), dtype=out_dtype, device=z.device)
+    _check(_tgt(z.data_ptr(), _rows(z), _i32(ids).data_ptr(), table.data_ptr(), table.stride(0), int(offset),
+                out.data_ptr(), T, n, _dt(z), _stream()), "token_gate")
+    return out
