@@ -412,6 +412,30 @@ def danipel_model(size: str, vocab: int = 32768, experts: int = 4, identity: int
                                    name=f"danipel-{size}")
 
 
+def tedenex_model(size: str, vocab: int = 32768, chunk: int = 512):
+    """Tedenex configuration of the same width, number of layer runs, head geometry and active
+    feed-forward parameters per token as ``hybrid_models(size)``: six layers (attention, time
+    mixing, latent attention, twice) of which the second and third run twice, i.e. eight layer
+    runs; attention over chunks of ``chunk`` tokens behind filters of 4 taps; time mixing with heads
+    of 64; latent attention with DeepSeek's proportions (latent of 512 + a rotated part of 64, heads
+    of 128 + 64 on the query side and 128 values, queries through a latent of 3 W / 8); dense
+    squared-relu feed-forward (2 * ff = 3 * intermediate) and a token input of W / 8 numbers per
+    layer."""
+    from minivllm_amd.models.tedenex import TedenexConfig
+    W, L, H, G, D, inter = HYBRID_SIZES[size]
+    mlp = {"kind": "dense", "ff": 3 * inter // 2}
+    kinds = [("attention", {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "conv": 4, "scale": D ** -0.5,
+                            "mask": {"size": chunk}}),
+             ("wkv", {"heads": W // 64, "dim": 64}),
+             ("latent_attention", {"heads": H, "dim": D, "rot_dim": 64, "vdim": D, "kv_rank": 512,
+                                   "q_rank": 3 * W // 8, "scale": (D + 64) ** -0.5,
+                                   "rot": {"base": 10000.0, "dims": 64}})]
+    layers = [{"type": kinds[i % 3][0], "mixer": kinds[i % 3][1], "mlp": mlp} for i in range(L - 2)]
+    return TedenexConfig.from_dict({"architecture": "Tedenex", "vocab": vocab, "width": W,
+                                    "norm": {"eps": 1e-6}, "token_side": {"dim": W // 8}, "layers": layers,
+                                    "loop": {"start": 1, "stop": 3, "times": 2}}, name=f"tedenex-{size}")
+
+
 def hybrid_comparison(args) -> dict:
     """Prefill and decode throughput of the hybrid families next to the dense decoder of the same
     size, one GPU, same engine path as the headline measurement (``bench_model``).
@@ -425,6 +449,8 @@ def hybrid_comparison(args) -> dict:
         return zegelix_comparison(args)
     if args.family == "danipel":
         return danipel_comparison(args)
+    if args.family == "tedenex":
+        return tedenex_comparison(args)
     out = {"metric": "prefill / decode tok/s, hybrid (attention + delta rule + routed experts) "
                      "next to the dense decoder of equal size",
            "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
@@ -555,6 +581,34 @@ def danipel_comparison(args) -> dict:
             if all(n in row and k in row[n] for n in ("danipel", "kidupel", "dense")):
                 row[f"danipel_over_kidupel_{k}"] = round(row["danipel"][k] / row["kidupel"][k], 3)
                 row[f"danipel_over_dense_{k}"] = round(row["danipel"][k] / row["dense"][k], 3)
+        out["sizes"][size] = row
+    return out
+
+
+def tedenex_comparison(args) -> dict:
+    out = {"metric": "prefill / decode tok/s, Tedenex (chunked attention behind filters, RWKV-style "
+                     "time mixing, latent attention, squared-relu feed-forward, token input per "
+                     "layer, looped stretch) next to Pelenex and the dense decoder of equal size",
+           "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+           "dtype": "bf16", "data": "synthetic random token prompts, random-init weights",
+           "config": {"seq_len": args.seq_len, "decode_batch": args.batch,
+                      "prefill_tokens_per_step": args.prefill_tokens, "kv_block_size": args.block_size},
+           "sizes": {}}
+    keep = ("prefill_tok_s", "prefill_ms_per_step", "decode_tok_s", "decode_ms_per_step",
+            "hipgraph_captured", "init_s")
+    for size in args.hybrid.split(","):
+        _, dense = hybrid_models(size)
+        row = {}
+        for name, make in (("tedenex", lambda: tedenex_model(size)), ("pelenex", lambda: pelenex_model(size)),
+                           ("dense", lambda: dense)):
+            if args.only and name != args.only:
+                continue                         # (a kernel trace of one model)
+            r = bench_model(args, make(), 0, 1)
+            row[name] = {k: (round(v, 3) if isinstance(v, float) else v) for k, v in r.items() if k in keep}
+        for k in ("prefill_tok_s", "decode_tok_s"):
+            if all(n in row and k in row[n] for n in ("tedenex", "pelenex", "dense")):
+                row[f"tedenex_over_pelenex_{k}"] = round(row["tedenex"][k] / row["pelenex"][k], 3)
+                row[f"tedenex_over_dense_{k}"] = round(row["tedenex"][k] / row["dense"][k], 3)
         out["sizes"][size] = row
     return out
 
@@ -858,12 +912,12 @@ def main():
                          "launch floor of a real N-GPU run; NOT a scaling number)")
     ap.add_argument("--p2p", action="store_true",
                     help="with --tp-shard: all-reduces by the peer-to-peer kernels in loop-back form")
-    ap.add_argument("--family", default="natilix", choices=["natilix", "pelenex", "kidupel", "zegelix", "danipel"],
+    ap.add_argument("--family", default="natilix", choices=["natilix", "pelenex", "kidupel", "zegelix", "danipel", "tedenex"],
                     help="with --hybrid: which hybrid family is measured (pelenex: next to natilix "
-                         "and dense; kidupel: next to pelenex and dense; zegelix, danipel: next to "
+                         "and dense; kidupel, tedenex: next to pelenex and dense; zegelix, danipel: next to "
                          "kidupel and dense)")
-    ap.add_argument("--only", default="", choices=["", "danipel", "zegelix", "kidupel", "pelenex", "natilix", "dense"],
-                    help="with --hybrid --family pelenex / kidupel / zegelix / danipel: measure this one model only")
+    ap.add_argument("--only", default="", choices=["", "tedenex", "danipel", "zegelix", "kidupel", "pelenex", "natilix", "dense"],
+                    help="with --hybrid --family pelenex / kidupel / zegelix / danipel / tedenex: measure this one model only")
     ap.add_argument("--hybrid", default="",
                     help="instead of the headline workload: the hybrid family (Natilix) next to "
                          "the dense decoder of equal size; comma-separated sizes of "

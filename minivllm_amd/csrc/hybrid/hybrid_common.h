@@ -62,12 +62,9 @@ __device__ __forceinline__ float siluf_(float z) { return z / (1.f + expf(-z)); 
 __device__ __forceinline__ float softplusf_(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 __device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.f + erff(z * 0.70710678118654752f)); }
 
-// sigmoid on the hardware exponential and reciprocal (both within a few ulp)
-__device__ __forceinline__ float fast_sigmoid(float z) { return __fdividef(1.f, 1.f + __expf(-z)); }
-
 // 0.5 z (1 + tanh(a)) = z sigmoid(2 a), a = sqrt(2/pi) (z + 0.044715 z^3)
 __device__ __forceinline__ float gelu_tanh_(float z) {
-    return z * fast_sigmoid(1.5957691216057308f * (z + 0.044715f * z * z * z));
+    return z * sigmoidf_(1.5957691216057308f * (z + 0.044715f * z * z * z));
 }
 
 // four (Vec4) or N (load_run, N % 4 == 0) consecutive elements widened to fp32; the address must

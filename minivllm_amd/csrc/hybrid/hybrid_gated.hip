@@ -272,6 +272,15 @@ __global__ void short_conv_kernel(const T* __restrict__ x, long x_stride, const 
     }
 }
 
+// sigmoid on the hardware exponential and reciprocal (both within a few ulp): the scan evaluates
+// three per element and pass
+__device__ __forceinline__ float fast_sigmoid(float z) { return __fdividef(1.f, 1.f + __expf(-z)); }
+
+// gelu_tanh_ on it
+__device__ __forceinline__ float fast_gelu_tanh(float z) {
+    return z * fast_sigmoid(1.5957691216057308f * (z + 0.044715f * z * z * z));
+}
+
 // 1 - exp(t) for t <= 0 without cancellation: the series next to zero, 1 - exp(t) elsewhere
 __device__ __forceinline__ float one_minus_exp(float t, float e) {
     const float series = -t * (1.f + t * (0.5f + t * (1.f / 6.f + t * (1.f / 24.f + t * (1.f / 120.f +
@@ -335,7 +344,7 @@ __global__ void rglru_scan_kernel(const float* __restrict__ u, const float* __re
     for (long t = lo; t < hi; ++t) {
         const GateStep g = rglru_step(gates, u, t, T_, C, c2, gcol, ch, br, bi, nsp);
         S = g.d * S + g.add;
-        if (live) st(out + t * C + ch, S * gelu_tanh_(ld(y + t * y_stride + ch)));
+        if (live) st(out + t * C + ch, S * fast_gelu_tanh(ld(y + t * y_stride + ch)));
     }
     if (wave == nw - 1 && live) state[(long)slot * C + ch] = S;
 }

@@ -22,6 +22,10 @@
 // MLSTM's running maximum is a sequential max-plus chain over tokens: wave 0 walks it once per
 // chunk (two dependent operations per token) and leaves the three factors of every token in LDS;
 // the normaliser n is kept by every lane group (its d-slice), since every column divides by n . q.
+// WKV's output is S^T q + (q . (u * k)) v: the factor of v is the same number for all columns and is
+// formed once per token, when a chunk has arrived in LDS, as ONE sum.  (A first token's output is
+// that number times v and is divided by its own root mean square afterwards: a number that suffers
+// from cancellation drops out again, which sums of their own in every column would not.)
 //
 // Sequence layout: `cu_q` [B+1] rows of each sequence (null: row b is sequence b), `positions`
 // (a sequence's first row holds the position its portion starts at; 0 = start from zeros),
@@ -64,8 +68,8 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
     constexpr int RS = NR + 4;                  // padded slice: neighbouring lanes hit different bank groups
     constexpr int IMG = CT * LPC * RS;          // floats of one [token][group lane][slice] image
     constexpr int NIMG = MODE == MLSTM ? 2 : 3; // k, q (, decay)
-    constexpr int NSC = MODE == MLSTM ? 3 : (MODE == CDELTA ? 1 : 0);    // LDS scalars per token
-    constexpr int NSC_IN = MODE == MLSTM ? 2 : NSC;                      // staged scalars per token
+    constexpr int NSC = MODE == MLSTM ? 3 : (MODE == GLA ? 0 : 1);       // LDS scalars per token
+    constexpr int NSC_IN = MODE == MLSTM ? 2 : (MODE == CDELTA ? 1 : 0); // staged scalars per token
     constexpr int BUF = NIMG * IMG + CT * COLS + NSC * CT;
     constexpr int IMG_ITEMS = CT * LPC * NR;
     constexpr int NITEM = NIMG * IMG_ITEMS + CT * COLS + NSC_IN * CT;
@@ -106,12 +110,6 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
     const TI* kp = (const TI*)a.k;
     const TI* vp = (const TI*)a.v;
 
-    float U[MODE == WKV ? NR : 1];
-    if constexpr (MODE == WKV) {
-#pragma unroll
-        for (int i = 0; i < NR; ++i) U[i] = d0 + i < D ? a.bonus[h * D + d0 + i] : 0.f;
-    }
-
     if (n == 1) {
         // A single token (decode rows, one-token portions): k, q and the decay vector of the head
         // (and MLSTM's three factors) are worked out once per workgroup into LDS, every lane then
@@ -145,6 +143,15 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
             }
         }
         __syncthreads();
+        if constexpr (MODE == WKV) {
+            if (tid < kWave) {
+                float dot = 0.f;
+                for (int d = tid; d < D; d += kWave) dot += sm[d] * sm[DP + d] * a.bonus[h * D + d];
+                dot = wave_sum(dot);
+                if (tid == 0) sm[NIMG * DP] = dot;
+            }
+            __syncthreads();
+        }
         float kk[NR], qq[NR], gg[MODE == MLSTM ? 1 : NR];
 #pragma unroll
         for (int i = 0; i < NR / 4; ++i) {
@@ -189,9 +196,8 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
         } else if constexpr (MODE == WKV) {
 #pragma unroll
             for (int i = 0; i < NR; ++i) {
-                const float kv = kk[i] * ve;
-                po += (S[i] + U[i] * kv) * qq[i];
-                S[i] = gg[i] * S[i] + kv;
+                po += S[i] * qq[i];
+                S[i] = gg[i] * S[i] + kk[i] * ve;
             }
         } else {
 #pragma unroll
@@ -208,6 +214,7 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
         if (col) {
             if (r == 0) {
                 if constexpr (MODE == MLSTM) po /= fmaxf(fabsf(pn), em) + 1e-6f;
+                if constexpr (MODE == WKV) po += sm[NIMG * LPC * NR] * ve;
                 a.o[(t * H + h) * (long)E + e] = po;
             }
 #pragma unroll
@@ -349,7 +356,25 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
             }
             __syncthreads();
         }
+        if constexpr (MODE == WKV) {                 // 16 neighbouring threads per token
+            const int tok = tid / 16;
+            if (tok < CT) {
+                const float* us = sm + 2 * BUF;
+                float dot = 0.f;
+#pragma unroll
+                for (int i = 0; i < LPC * NR / 16; ++i) {
+                    const int d = tid % 16 + 16 * i, at = (tok * LPC + d / NR) * RS + d % NR;
+                    dot += buf[at] * buf[IMG + at] * us[d];
+                }
+#pragma unroll
+                for (int x = 1; x < 16; x <<= 1) dot += __shfl_xor(dot, x, kWave);
+                if (tid % 16 == 0) buf[NIMG * IMG + CT * COLS + tok] = dot;
+            }
+            __syncthreads();
+        }
     };
+    if constexpr (MODE == WKV)
+        for (int d = tid; d < LPC * NR; d += 256) sm[2 * BUF + d] = d < D ? a.bonus[h * D + d] : 0.f;
     TI reg[NLD];
     fetch(0, reg);
     stash(0, reg, sm);
@@ -423,9 +448,8 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
                     } else if constexpr (MODE == WKV) {
 #pragma unroll
                         for (int i = 0; i < NR; ++i) {
-                            const float kv = kk[i] * ve;
-                            o4[i & 3] += (S[i] + U[i] * kv) * qq[i];
-                            S[i] = gg[i] * S[i] + kv;
+                            o4[i & 3] += S[i] * qq[i];
+                            S[i] = gg[i] * S[i] + kk[i] * ve;
                         }
                     } else {
 #pragma unroll
@@ -451,6 +475,7 @@ __global__ void __launch_bounds__(256) gated_scan_kernel(const ScanArgs a) {
                 const int tok = tb + j;
                 if (tok < nt && col && r == j) {
                     float out = po[j];
+                    if constexpr (MODE == WKV) out += sc[tok] * buf[NIMG * IMG + tok * COLS + c];
                     if constexpr (MODE == MLSTM) out /= fmaxf(fabsf(pn[j]), sc[2 * CT + tok]) + 1e-6f;
                     a.o[((first + ch * CT + tok) * H + h) * (long)E + e] = out;
                 }
@@ -480,10 +505,11 @@ static void launch_scan(const ScanArgs& a, int B, hipStream_t s) {
     constexpr int CT = NR >= 64 ? 8 : 16;
     constexpr int COLS = 256 / LPC;
     constexpr int NIMG = MODE == MLSTM ? 2 : 3;
-    constexpr int NSC = MODE == MLSTM ? 3 : (MODE == CDELTA ? 1 : 0);
+    constexpr int NSC = MODE == MLSTM ? 3 : (MODE == GLA ? 0 : 1);
     constexpr int BUF = NIMG * CT * LPC * (NR + 4) + CT * COLS + NSC * CT;
+    constexpr int BONUS = MODE == WKV ? LPC * NR : 0;
     hipLaunchKernelGGL((gated_scan_kernel<TI, NR, LPC, MODE>), dim3(B, a.H, (a.E + COLS - 1) / COLS),
-                       dim3(256), 2 * BUF * sizeof(float), s, a);
+                       dim3(256), (2 * BUF + BONUS) * sizeof(float), s, a);
 }
 
 // Lanes per state column: the fewest of 4 / 8 / 16 that give every CU a workgroup

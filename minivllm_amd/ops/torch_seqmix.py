@@ -826,14 +826,13 @@ def wkv_scan(r, k, v, w_raw, w_bias, bonus, state, cu_q, positions, slots):
     E = v.shape[2]
     rf, kf, vf = r.float(), k.float(), v.float()
     decay = torch.exp(-torch.exp(w_raw.float().reshape(T, H, D) + w_bias.float().view(H, D)))
-    u = bonus.float().view(H, D, 1)
+    dot = (rf * kf * bonus.float().view(H, D)).sum(-1, keepdim=True)          # [T, H, 1]
     o = torch.zeros(T, H, E, dtype=torch.float32)
     for s, e, slot, past in _seq_rows(cu_q, positions, slots):
         S = state[slot].clone() if past else torch.zeros(H, D, E)
         for t in range(s, e):
-            kv = kf[t][:, :, None] * vf[t][:, None, :]
-            o[t] = torch.einsum("hde,hd->he", S + u * kv, rf[t])
-            S = decay[t][:, :, None] * S + kv
+            o[t] = torch.einsum("hde,hd->he", S, rf[t]) + dot[t] * vf[t]
+            S = decay[t][:, :, None] * S + kf[t][:, :, None] * vf[t][:, None, :]
         state[slot] = S
     return o
 

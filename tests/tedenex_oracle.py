@@ -41,11 +41,9 @@ def time_filter(u, w):
     """u [T, C], w [C, taps]: y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros before the start."""
     taps = w.shape[1]
     y = torch.zeros_like(u)
-    for t in range(u.shape[0]):
-        for j in range(taps):
-            s = t - (taps - 1) + j
-            if s >= 0:
-                y[t] += w[:, j] * u[s]
+    for j in range(taps):
+        back = taps - 1 - j
+        y[back:] += w[:, j] * u[:max(u.shape[0] - back, 0)]
     return y
 
 
@@ -58,15 +56,13 @@ def attention(h, w, m, eps):
     q = unit_rms(q.view(T, H, D), eps) * w["q.norm"]
     k = unit_rms(k.view(T, G, D), eps) * w["k.norm"]
     v = v.view(T, G, E)
+    i, j = torch.arange(T)[:, None], torch.arange(T)[None, :]
+    hidden = (j > i) | (torch.div(i, size, rounding_mode="floor") != torch.div(j, size, rounding_mode="floor"))
     out = torch.zeros(T, H, E, dtype=F64)
     for hd in range(H):
         g = hd // (H // G)
-        slope = 2.0 ** (-8.0 * (hd + 1) / H)
-        for i in range(T):
-            lo = i // size * size
-            j = torch.arange(lo, i + 1)
-            s = (k[lo:i + 1, g] @ q[i, hd]) * float(m["scale"]) - slope * (i - j).to(F64)
-            out[i, hd] = torch.softmax(s, 0) @ v[lo:i + 1, g]
+        s = q[:, hd] @ k[:, g].T * float(m["scale"]) - 2.0 ** (-8.0 * (hd + 1) / H) * (i - j)
+        out[:, hd] = torch.softmax(s.masked_fill(hidden, float("-inf")), -1) @ v[:, g]
     return out.reshape(T, H * E) @ w["o"].T
 
 
