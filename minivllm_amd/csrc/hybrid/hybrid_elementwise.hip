@@ -193,6 +193,36 @@ __global__ void gated_head_norm_kernel(const float* __restrict__ o, const float*
     }
 }
 
+// The same with LPH neighbouring lanes per head, eight columns each (E <= 8 LPH, whole runs);
+// `heads` = T * H heads in all.
+template <typename T, int LPH>
+__global__ void __launch_bounds__(256)
+gated_head_norm_runs_kernel(const float* __restrict__ o, const float* __restrict__ w,
+                            const T* __restrict__ gate, long gate_stride, T* __restrict__ out, long heads,
+                            int H, int E, float eps, int w_heads, int sig) {
+    const long th = blockIdx.x * (long)(256 / LPH) + threadIdx.x / LPH;
+    const int e = (threadIdx.x % LPH) * 8;
+    if (th >= heads) return;                             // (whole groups leave)
+    const long t = th / H;
+    const int h = (int)(th - t * H);
+    const bool live = e < E;
+    float v[8], z[8], wv[8], s = 0.f;
+    if (live) {
+        load_run<float, 8>(o + th * E + e, v);
+        load_run<T, 8>(gate + t * gate_stride + (long)h * E + e, z);
+        load_run<float, 8>(w + (w_heads ? (long)h * E : 0) + e, wv);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) s += v[i] * v[i];
+    }
+#pragma unroll
+    for (int x = 1; x < LPH; x <<= 1) s += __shfl_xor(s, x, kWave);
+    if (!live) return;
+    const float r = rsqrtf(s / (float)E + eps);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] *= r * wv[i] * (sig ? sigmoidf_(z[i]) : siluf_(z[i]));
+    store_run8<T>(out + th * E + e, v);
+}
+
 // One workgroup (256 threads) per token: fp32 router logits (the row is read once, eight experts'
 // partial sums per pass), softmax over all experts (sig: the sigmoid of each logit instead), best
 // `keep` of `groups` groups (a group scores its best expert), `top` largest eligible scores; dense
@@ -365,6 +395,22 @@ int hyb_gated_head_norm(const void* o, const void* w, const void* gate, long gat
                         void* out, long T_, int H, int E, float eps, int w_heads, int sig, int dt,
                         hipStream_t s) {
     if (T_ <= 0) return 0;
+#define GHN_RUNS(LPH)                                                                              \
+    HYB_DISPATCH(dt, hipLaunchKernelGGL((gated_head_norm_runs_kernel<T, LPH>),                     \
+                                        dim3((unsigned)((T_ * H + 256 / LPH - 1) / (256 / LPH))),  \
+                                        dim3(256), 0, s, (const float*)o, (const float*)w,         \
+                                        (const T*)gate, gate_stride, (T*)out, T_ * H, H, E, eps,   \
+                                        w_heads, sig))
+    if (E % 8 == 0 && E <= 512 && gate_stride % 8 == 0 &&
+        ((size_t)o | (size_t)w | (size_t)gate | (size_t)out) % 16 == 0) {
+        if (E <= 32) GHN_RUNS(4);
+        else if (E <= 64) GHN_RUNS(8);
+        else if (E <= 128) GHN_RUNS(16);
+        else if (E <= 256) GHN_RUNS(32);
+        else GHN_RUNS(64);
+        return HYB_LAUNCH_OK();
+    }
+#undef GHN_RUNS
     HYB_DISPATCH(dt, hipLaunchKernelGGL(gated_head_norm_kernel<T>, dim3(T_ * H), dim3(kWave), 0, s,
                                         (const float*)o, (const float*)w, (const T*)gate,
                                         gate_stride, (T*)out, H, E, eps, w_heads, sig));

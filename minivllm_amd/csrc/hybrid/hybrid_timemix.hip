@@ -16,22 +16,24 @@
 
 using namespace hyb;
 
+// Where row t (the same for every lane of a wave) stands.
 struct RowPlace {
     int slot, off, pos;      // state slot (< 0: none), index inside the portion, position
     bool single;             // the only row of its sequence in this step
+    RowPlace() = default;
     __device__ __forceinline__ RowPlace(long t, const int* cu_q, const int* positions, const int* slots,
                                         const int* row_seq) {
-        const int b = cu_q ? row_seq[t] : (int)t;
-        slot = b >= 0 ? slots[b] : -1;
-        off = 0; pos = 0; single = true;
-        if (slot < 0) return;
-        if (cu_q) {
-            const int s0 = cu_q[b];
+        const int b = cu_q ? uniform(row_seq[t]) : (int)t;
+        slot = b >= 0 ? uniform(slots[b]) : -1;
+        pos = uniform(positions[t]);
+        off = 0; single = true;
+        if (cu_q && b >= 0) {
+            const int s0 = uniform(cu_q[b]);
             off = (int)t - s0;
-            single = cu_q[b + 1] - s0 == 1;
+            single = uniform(cu_q[b + 1]) - s0 == 1;
         }
-        pos = positions[t];
     }
+    static __device__ __forceinline__ int uniform(int v) { return __builtin_amdgcn_readfirstlane(v); }
 };
 
 struct FilterArgs {
@@ -45,13 +47,39 @@ struct FilterArgs {
     float eps;
 };
 
+// eight elements as they are in memory, widened when they are needed
+template <typename T> struct Raw8;
+template <> struct Raw8<bf16_t> {
+    uint4 v;
+    __device__ __forceinline__ void load(const bf16_t* p) { v = *reinterpret_cast<const uint4*>(p); }
+    __device__ __forceinline__ void widen(float* o) const {
+        const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            o[2 * i] = __uint_as_float(w[i] << 16);
+            o[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
+        }
+    }
+};
+template <> struct Raw8<float> {
+    float4 a, b;
+    __device__ __forceinline__ void load(const float* p) {
+        a = *reinterpret_cast<const float4*>(p);
+        b = *reinterpret_cast<const float4*>(p + 4);
+    }
+    __device__ __forceinline__ void widen(float* o) const {
+        o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w;
+        o[4] = b.x; o[5] = b.y; o[6] = b.z; o[7] = b.w;
+    }
+};
+
 // A group of LPH neighbouring lanes owns one head (q heads first, then k, then v), eight channels per
-// lane, and walks `rows_per` rows with the filter's window in registers: an input is loaded once per
-// group of rows.  grid (row groups, groups of 256 / LPH heads).
-template <typename T, int TAPS, int LPH>
+// lane, and walks ROWS rows, whose inputs are all requested ahead, with the filter's window in
+// registers: an input is loaded once per group of rows.  grid (row groups, groups of 256 / LPH heads).
+template <typename T, int TAPS, int LPH, int ROWS>
 __global__ void __launch_bounds__(256)
 conv_norm_store_kernel(const T* __restrict__ x, const FilterArgs a, T* __restrict__ q_out,
-                       T* __restrict__ k_cache, T* __restrict__ v_cache, int rows_per) {
+                       T* __restrict__ k_cache, T* __restrict__ v_cache) {
     const int hd = blockIdx.y * (256 / LPH) + threadIdx.x / LPH, d = (threadIdx.x % LPH) * 8;
     const int H = a.H, G = a.G, D = a.D, E = a.E;
     if (hd >= H + 2 * G) return;                             // (whole groups leave)
@@ -59,6 +87,19 @@ conv_norm_store_kernel(const T* __restrict__ x, const FilterArgs a, T* __restric
     const int n = isv ? E : D;
     const int c = (isv ? (H + G) * D + (hd - H - G) * E : hd * D) + d;
     const bool live = d < n;
+    const long t0 = (long)blockIdx.x * ROWS;
+    Raw8<T> in[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r)
+        if (live && t0 + r < a.T_) in[r].load(x + (t0 + r) * a.x_stride + c);
+    RowPlace places[ROWS];
+    int rows[ROWS];                                          // cache row of each
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) {
+        const long t = min(t0 + r, a.T_ - 1);
+        places[r] = RowPlace(t, a.cu_q, a.positions, a.slots, a.row_seq);
+        rows[r] = a.slot_mapping ? RowPlace::uniform(a.slot_mapping[t]) : -1;
+    }
     float w[8][TAPS], gain[8], hist[TAPS > 1 ? TAPS - 1 : 1][8];
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
@@ -67,10 +108,11 @@ conv_norm_store_kernel(const T* __restrict__ x, const FilterArgs a, T* __restric
         for (int j = 0; j < TAPS; ++j) w[i][j] = live ? a.w[(long)(c + i) * TAPS + j] : 0.f;
     }
     bool fresh = true;                                       // the window is not this row's
-    for (int r = 0; r < rows_per; ++r) {
-        const long t = (long)blockIdx.x * rows_per + r;
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) {
+        const long t = t0 + r;
         if (t >= a.T_) return;
-        const RowPlace at(t, a.cu_q, a.positions, a.slots, a.row_seq);
+        const RowPlace& at = places[r];
         if (at.slot < 0) {
             fresh = true;
             if (isq && live) {
@@ -83,7 +125,7 @@ conv_norm_store_kernel(const T* __restrict__ x, const FilterArgs a, T* __restric
         float cur[8], y[8];
 #pragma unroll
         for (int i = 0; i < 8; ++i) cur[i] = 0.f;
-        if (live) load_run<T, 8>(x + t * a.x_stride + c, cur);
+        if (live) in[r].widen(cur);
         if (fresh || at.off == 0) {
 #pragma unroll
             for (int j = 0; j < TAPS - 1; ++j) {
@@ -115,7 +157,7 @@ conv_norm_store_kernel(const T* __restrict__ x, const FilterArgs a, T* __restric
         if (live) {
             if (isq) store_run8<T>(q_out + (t * H + hd) * (long)D + d, y);
             else {
-                const long slot = a.slot_mapping ? a.slot_mapping[t] : -1;
+                const long slot = rows[r];
                 if (slot >= 0 && k_cache) {
                     if (isv) store_run8<T>(v_cache + (slot * G + hd - H - G) * (long)E + d, y);
                     else store_run8<T>(k_cache + (slot * G + hd - H) * (long)D + d, y);
@@ -317,12 +359,16 @@ int hyb_conv_norm_store(const void* x, long x_stride, const void* w, void* tail,
     const size_t align = (size_t)x | (size_t)tail | (size_t)q_out | (size_t)k_cache | (size_t)v_cache;
     const bool runs = D % 8 == 0 && E % 8 == 0 && longest <= 512 && x_stride % 8 == 0 && align % 16 == 0;
     int own = 0;                                             // the kernel keeps single rows' inputs
-    const int rows_per = T_ >= 2048 ? 8 : 1;
-#define FILTER(TAPS, LPH)                                                                          \
-    HYB_DISPATCH(dt, hipLaunchKernelGGL((conv_norm_store_kernel<T, TAPS, LPH>),                    \
-                                        dim3((unsigned)((T_ + rows_per - 1) / rows_per),           \
+#define FILTER_ROWS(TAPS, LPH, ROWS)                                                               \
+    HYB_DISPATCH(dt, hipLaunchKernelGGL((conv_norm_store_kernel<T, TAPS, LPH, ROWS>),              \
+                                        dim3((unsigned)((T_ + ROWS - 1) / ROWS),                   \
                                              (heads + 256 / LPH - 1) / (256 / LPH)), dim3(256), 0, s, \
-                                        (const T*)x, a, (T*)q_out, (T*)k_cache, (T*)v_cache, rows_per))
+                                        (const T*)x, a, (T*)q_out, (T*)k_cache, (T*)v_cache))
+#define FILTER(TAPS, LPH)                                        \
+    do {                                                         \
+        if (T_ >= 2048) FILTER_ROWS(TAPS, LPH, 8);               \
+        else FILTER_ROWS(TAPS, LPH, 1);                          \
+    } while (0)
 #define FILTER_TAPS(TAPS)                              \
     do {                                               \
         if (longest <= 64) FILTER(TAPS, 8);            \
@@ -343,6 +389,7 @@ int hyb_conv_norm_store(const void* x, long x_stride, const void* w, void* tail,
     }
 #undef FILTER_TAPS
 #undef FILTER
+#undef FILTER_ROWS
     if (hipGetLastError() != hipSuccess) return 2;
     if (taps > 1 && B > 0 && (cu_q || !own))
         HYB_DISPATCH(dt, launch_tail<T>(x, x_stride, tail, cu_q, positions, slots, B, a.C, taps, own, s));

@@ -295,3 +295,15 @@ def test_steps_in_a_captured_graph():
                 assert torch.equal(g_[live], w_[live])
         for s, t in zip(a, b):
             assert torch.equal(s, t)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,E,T", [(16, 64, 33), (3, 24, 7), (5, 128, 4), (2, 200, 9), (1, 512, 3), (4, 9, 5), (2, 520, 2)])
+@pytest.mark.parametrize("act", ["silu", "sigmoid"])
+@pytest.mark.parametrize("per_head", [True, False])
+def test_gated_head_norm(dt, H, E, T, act, per_head):
+    torch.manual_seed(E)
+    o, w = torch.randn(T, H, E), torch.randn(H * E if per_head else E)
+    gate = torch.randn(T, H * E + 8).to(dt)[:, :H * E]
+    torch.testing.assert_close(hk.gated_head_norm(o.cuda(), w.cuda(), gate.cuda(), 1e-4, dt, act).cpu().float(),
+                               ref.gated_head_norm(o, w, gate, 1e-4, dt, act).float(), **tol(dt))
